@@ -5,7 +5,10 @@ The shared library is built in-tree (``axonml_amd/libaxq.so``) by
 or CPU fallback: if the library is missing, loading raises.
 """
 import ctypes as C
+import fcntl
 import os
+import subprocess
+import sys
 
 _HERE = os.path.dirname(os.path.abspath(__file__))
 LIB_PATH = os.path.join(_HERE, "libaxq.so")
@@ -55,6 +58,18 @@ class ModelConfig(C.Structure):
     ]
 
 
+class LayerConfig(C.Structure):
+    _fields_ = [("mixer", C.c_int32), ("heads", C.c_int32), ("kv_heads", C.c_int32), ("dim", C.c_int32), ("vdim", C.c_int32), ("ff", C.c_int32),
+                ("bias_rows", C.c_int32), ("bias_max", C.c_int32), ("q_temp_every", C.c_int32), ("q_temp_coef", C.c_float), ("scale", C.c_float),
+                ("decay_rank", C.c_int32)]
+
+
+class StackConfig(C.Structure):
+    _fields_ = [("vocab_size", C.c_int32), ("width", C.c_int32), ("max_positions", C.c_int32), ("cache_positions", C.c_int32),
+                ("num_layers", C.c_int32), ("loop_start", C.c_int32), ("loop_stop", C.c_int32), ("loop_times", C.c_int32), ("compute", C.c_int32),
+                ("norm_eps", C.c_float), ("logit_softcap", C.c_float), ("layers", C.POINTER(LayerConfig))]
+
+
 _vp, _sz, _i, _i64 = C.c_void_p, C.c_size_t, C.c_int, C.c_int64
 
 # name -> (restype, argtypes): every symbol include/axq.h declares.
@@ -101,6 +116,10 @@ SIGNATURES = {
     "axq_model_reset": (_i, [_vp]),
     "axq_model_forward": (_i, [_vp, C.c_int32, _vp, C.POINTER(C.c_int32)]),
     "axq_model_forward_tokens": (_i, [_vp, _vp, _i, _vp, C.POINTER(C.c_int32)]),
+    "axq_model_forward_rows": (_i, [_vp, _vp, _i, _vp, _i, _vp, _vp]),
+    "axq_model_layer_runs": (_i, [_vp]),
+    "axq_model_create_stack": (_i, [_vp, C.POINTER(StackConfig), C.POINTER(_vp)]),
+    "axq_model_set_tensor": (_i, [_vp, _i, C.c_char_p, _vp, _i64, _i64]),
     "axq_model_generate": (_i, [_vp, _vp, _i, _i, _vp, C.POINTER(C.c_float), C.POINTER(C.c_float)]),
     "axq_model_seq_len": (_i, [_vp]),
     "axq_model_set_batch": (_i, [_vp, _i]),
@@ -131,6 +150,19 @@ SIGNATURES = {
 }
 
 _lib = None
+
+
+def build_library():
+    """Compiles libaxq.so where it is missing (programs that must work in a fresh checkout call this first).  Callers that
+    come at the same time wait for the one that compiles."""
+    if os.path.exists(LIB_PATH):
+        return
+    src = os.path.join(_HERE, "csrc")
+    with open(os.path.join(src, "Makefile")) as lock:
+        fcntl.flock(lock, fcntl.LOCK_EX)
+        if not os.path.exists(LIB_PATH):
+            jobs = min(16, len(os.sched_getaffinity(0)))
+            subprocess.run(["make", "-C", src, "-s", f"-j{jobs}"], check=True, stdout=sys.stderr)
 
 
 def load_library():

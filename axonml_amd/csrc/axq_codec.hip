@@ -454,6 +454,21 @@ __global__ void dequant_f16_kernel(const uint16_t *src, size_t numel, float *out
     }
 }
 
+// ---- BF16: the upper half of the f32, rounded to nearest even; NaN stays NaN
+__device__ inline uint16_t f32_to_bf16_bits(float f) {
+    const uint32_t u = __builtin_bit_cast(uint32_t, f);
+    if ((u & 0x7FFFFFFFu) > 0x7F800000u) return (uint16_t)((u >> 16) | 0x40u);
+    return (uint16_t)((u + 0x7FFFu + ((u >> 16) & 1u)) >> 16);
+}
+__global__ void quant_bf16_kernel(const float *src, size_t numel, uint16_t *out) {
+    const size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
+    if (i < numel) out[i] = f32_to_bf16_bits(src[i]);
+}
+__global__ void dequant_bf16_kernel(const uint16_t *src, size_t numel, float *out) {
+    const size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
+    if (i < numel) out[i] = __builtin_bit_cast(float, (uint32_t)src[i] << 16);
+}
+
 // ---- dequantisers: dequantize.rs:89-92, 116-121, 145-151 -------------------
 // One thread per 32 elements; for Q4_K a thread handles one sub-block.
 // The 32 values of a thread go through an LDS tile (rows padded to 33 floats), so that the workgroup's 16 KB of
@@ -785,6 +800,7 @@ int axq_dev_quantize(axq_ctx *ctx, int type, const float *src, size_t numel, uin
     case AXQ_Q5_K: quant_qk_kernel<5><<<grid_for(nblk * 8, B), B, 0, ctx->stream>>>(src, numel, nblk, packed); break;
     case AXQ_Q6_K: quant_q6_k_kernel<<<grid_for(nblk * 16, B), B, 0, ctx->stream>>>(src, numel, nblk, packed); break;
     case AXQ_F16: quant_f16_kernel<<<grid_for((numel + 7) / 8, 256), 256, 0, ctx->stream>>>(src, numel, (uint16_t *)packed); break;
+    case AXQ_BF16: quant_bf16_kernel<<<grid_for(numel, 256), 256, 0, ctx->stream>>>(src, numel, (uint16_t *)packed); break;
     case AXQ_F32:
         AXQ_HIP(ctx, hipMemcpyAsync(packed, src, numel * 4, hipMemcpyDeviceToDevice, ctx->stream), AXQ_ERR_COPY_FAILED);
         return AXQ_OK;
@@ -805,6 +821,7 @@ int axq_dev_dequantize(axq_ctx *ctx, int type, const uint8_t *packed, size_t num
     case AXQ_F16:
         dequant_f16_kernel<<<grid_for((numel + 7) / 8, 256), 256, 0, ctx->stream>>>((const uint16_t *)packed, numel, dst);
         break;
+    case AXQ_BF16: dequant_bf16_kernel<<<grid_for(numel, 256), 256, 0, ctx->stream>>>((const uint16_t *)packed, numel, dst); break;
     case AXQ_F32:
         AXQ_HIP(ctx, hipMemcpyAsync(dst, packed, numel * 4, hipMemcpyDeviceToDevice, ctx->stream), AXQ_ERR_COPY_FAILED);
         return AXQ_OK;
@@ -819,6 +836,13 @@ int axq_dev_repack(axq_ctx *ctx, const axq_weight *w, uint8_t *packed, bool to_p
         void *dst = to_planar ? (void *)w->codes : (void *)packed;
         const void *src = to_planar ? (const void *)packed : (const void *)w->codes;
         AXQ_HIP(ctx, hipMemcpyAsync(dst, src, w->packed_bytes, hipMemcpyDeviceToDevice, ctx->stream), AXQ_ERR_COPY_FAILED);
+        return AXQ_OK;
+    }
+    if (w->type == AXQ_BF16) { // rows padded to w->codes_pitch (the padding stays zero)
+        const size_t row = (size_t)w->k * 2;
+        AXQ_HIP(ctx, to_planar ? hipMemcpy2DAsync(w->codes, w->codes_pitch, packed, row, row, (size_t)w->n_rows, hipMemcpyDeviceToDevice, ctx->stream)
+                               : hipMemcpy2DAsync(packed, row, w->codes, w->codes_pitch, row, (size_t)w->n_rows, hipMemcpyDeviceToDevice, ctx->stream),
+                AXQ_ERR_COPY_FAILED);
         return AXQ_OK;
     }
     PlanarDesc d;

@@ -22,56 +22,8 @@
 #include <vector>
 
 #include "axq_internal.h"
+#include "axq_model.h"
 #include "axq_split.h"
-
-struct axq_model {
-    axq_ctx *ctx;
-    axq_model_config cfg;
-    int qkv_rows, q_dim, kv_dim;
-    // weights
-    uint16_t *emb;                  // f16 [vocab, hidden], or
-    float *emb32 = nullptr;         // f32 [vocab, hidden] as the reference keeps it (one of the two is set)
-    float *norm_attn, *norm_ffn;    // [layers, hidden]
-    float *norm_final;              // [hidden]
-    std::vector<axq_weight *> w_qkv, w_o, w_gu, w_down;
-    // q, k or v of a layer whose block type differs from the fused weight's (GGUF files that keep attn_v at six bits
-    // beside four-bit attn_q and attn_k): a weight of its own, multiplied after the fused one into its rows of qkv
-    std::vector<axq_weight *> w_sep[3];
-    axq_weight *w_head;
-    std::vector<uint32_t> set_mask; // per layer: bit per axq_linear_id that has been set
-    bool head_set;
-    float *rope_cos, *rope_sin;     // [max_pos, head_dim / 2]
-    uint16_t *kcache, *vcache;      // f16 [layers, kv_heads, max_pos, head_dim]
-    // activations
-    float *h, *xn, *qkv, *att, *gu, *act, *logits;
-    float *att_part;                // [kv_heads][max_splits][rep][head_dim + 2] partial attention results
-    float *pb_h, *pb_xn, *pb_qkv, *pb_att, *pb_gu, *pb_act; // the same activations for pb_cap prompt tokens at a time
-    int pb_cap;
-    int n_seq;                      // sequences the caches and the per-sequence state hold (axq_model_set_batch)
-    size_t seq_stride;              // cache elements of one sequence: layers * kv_heads * max_pos * head_dim
-    size_t part_stride;             // floats of att_part per sequence
-    std::vector<int> seq_pos;       // host mirror of pos[s] for the batched calls (sequence 0: host_pos)
-    int32_t *bprompt, *boffsets, *bout; // prompts, their offsets and the generated ids of a batched generate
-    hipGraphExec_t graph_b, graph_bf; // batched step: split attention / one attention workgroup per head (short contexts)
-    bool graph_b_ok, graph_bf_ok;
-    int max_splits;
-    // device-side state
-    int32_t *pos, *tok, *next, *gen, *prompt, *out;
-    int32_t *hist;                  // every token fed so far, by position (what a repetition penalty looks at)
-    void *sample_scratch;           // scratch of the sampler, allocated when one is set
-    bool sampling;                  // next token by axq_sampling_config instead of the plain argmax
-    axq_sampling_config sampler;
-    uint64_t sample_seed;
-    int prompt_cap, out_cap;
-    int host_pos;
-    hipGraphExec_t graph;           // the one-token step with the attention split over the positions
-    bool graph_ok;
-    hipGraphExec_t graph_f;         // the same with one attention workgroup per head (short contexts)
-    bool graph_f_ok;
-    int fused_max;                  // contexts up to this many positions take graph_f
-    int prompt_chunk;               // most prompt rows per pass through the layers
-    bool attn_mfma;                 // prompt attention of many rows on the matrix pipe (development knob AXQ_ATTN_MFMA=0: off)
-};
 
 namespace {
 
@@ -833,6 +785,13 @@ size_t prompt_attn_lds(const axq_model *m, int last);
 // and value included); otherwise the positions are split over workgroups and a second kernel merges them.
 int enqueue_step(axq_model *m, bool short_ctx) {
     axq_ctx *ctx = m->ctx;
+    if (m->stack) {
+        int e = axq_stack_step(m);
+        if (e) return e;
+        argmax_kernel<<<1, 1024, 0, ctx->stream>>>(m->logits, m->cfg.vocab_size, m->next, m->pos);
+        AXQ_LAUNCH_CHECK(ctx, "decode step");
+        return AXQ_OK;
+    }
     const axq_model_config &c = m->cfg;
     hipStream_t st = ctx->stream;
     const int H = c.hidden_size;
@@ -864,6 +823,7 @@ int enqueue_step(axq_model *m, bool short_ctx) {
 }
 
 int check_ready(axq_model *m) {
+    if (m->stack) return axq_stack_ready(m);
     if ((!m->emb && !m->emb32) || !m->head_set) return axq_fail(m->ctx, AXQ_ERR_INVALID_DATA, "Invalid quantized data: embedding or lm_head not set");
     for (int l = 0; l < m->cfg.num_hidden_layers; l++)
         if (m->set_mask[l] != (1u << AXQ_LIN_COUNT) - 1)
@@ -875,7 +835,7 @@ int check_ready(axq_model *m) {
 // Captures the step into a graph on first use; later calls replay it.  pos: the position of the token being fed.
 int run_step_graph(axq_model *m, int pos) {
     axq_ctx *ctx = m->ctx;
-    const bool short_ctx = pos < m->fused_max;
+    const bool short_ctx = !m->stack && pos < m->fused_max;
     static const bool no_graph = getenv("AXQ_DECODE_GRAPH") && getenv("AXQ_DECODE_GRAPH")[0] == '0';
     if (no_graph) return enqueue_step(m, short_ctx); // development knob: plain launches instead of a graph replay
     hipGraphExec_t &exec = short_ctx ? m->graph_f : m->graph;
@@ -1125,11 +1085,56 @@ int enqueue_rows(axq_model *m, const Rows &r) {
 
 // Feeds toks[0..n) (device memory) to sequence `seq` from position pos0 on as rows, several at a time; returns how many
 // went in (all, unless the attention scores of so long a context do not fit LDS: then none from there on).
-int feed_rows(axq_model *m, int seq, const int32_t *toks, int n, int pos0, int *fed) {
+// Logits of chosen tokens of a call (axq_model_forward_rows).
+struct Wanted {
+    const int32_t *places; // host, rising
+    int n, total;          // how many; tokens of the call
+    float *logits;         // host, [n][vocab]
+    float *layers;         // host, [layer runs][total][hidden], or NULL
+};
+
+// The wanted logits among the nb rows that just went through the layers (row 0 is token i of the call).
+int wanted_logits(axq_model *m, const Wanted *w, int i, int nb) {
+    if (!w) return AXQ_OK;
+    axq_ctx *ctx = m->ctx;
+    std::vector<int32_t> rows;
+    int first = -1;
+    for (int j = 0; j < w->n; j++)
+        if (w->places[j] >= i && w->places[j] < i + nb) {
+            if (first < 0) first = j;
+            rows.push_back(w->places[j] - i);
+        }
+    if (rows.empty()) return AXQ_OK;
+    const size_t V = (size_t)m->cfg.vocab_size;
+    float *dst = w->logits + (size_t)first * V;
+    if (m->stack) return axq_stack_logits_rows(m, rows.data(), (int)rows.size(), dst);
+    const int H = m->cfg.hidden_size;
+    for (size_t j = 0; j < rows.size(); j++) {
+        norm_kernel<<<1, 1024, 0, ctx->stream>>>(m->pb_h + (size_t)rows[j] * H, m->norm_final, H, m->cfg.rms_norm_eps, m->pb_xn);
+        int rc = axq_dev_gemv(ctx, m->w_head, m->pb_xn, 1, nullptr, m->logits);
+        if (rc) return rc;
+        AXQ_HIP(ctx, hipMemcpyAsync(dst + j * V, m->logits, V * 4, hipMemcpyDeviceToHost, ctx->stream), AXQ_ERR_COPY_FAILED);
+    }
+    return AXQ_OK;
+}
+
+int feed_rows(axq_model *m, int seq, const int32_t *toks, int n, int pos0, int *fed, const Wanted *w = nullptr) {
     static const char *knob = getenv("AXQ_PROMPT_BATCH"); // development knob: 0 = no rows at all, 1 = no GEMM
     const int allow = knob ? atoi(knob) : 2;
     int i = 0, rc;
     *fed = 0;
+    while (m->stack && i < n) { // rows of any number go through described layers together
+        const int nb = n - i < m->prompt_chunk ? n - i : m->prompt_chunk, p0 = pos0 + i;
+        for (int t0 = 0; t0 < nb; t0 += 1024)
+            record_tokens_kernel<<<1, nb - t0 < 1024 ? nb - t0 : 1024, 0, m->ctx->stream>>>(m->hist, p0 + t0, toks + i + t0);
+        if (w) axq_stack_trace(m, w->layers, w->total, i);
+        if ((rc = axq_stack_rows(m, toks + i, nb, p0))) return rc;
+        add_i32_kernel<<<1, 1, 0, m->ctx->stream>>>(m->pos, nb);
+        if ((rc = wanted_logits(m, w, i, nb))) return rc;
+        i += nb;
+        *fed = i;
+    }
+    if (m->stack) return AXQ_OK;
     while (allow >= 1 && i < n) {
         const int left = n - i;
         Rows r;
@@ -1147,6 +1152,7 @@ int feed_rows(axq_model *m, int seq, const int32_t *toks, int n, int pos0, int *
         r.lds = prompt_attn_lds(m, r.pos0 + r.nb);
         if ((rc = reserve_prompt_rows(m, r.nb))) return rc;
         if ((rc = enqueue_rows(m, r))) return rc;
+        if ((rc = wanted_logits(m, w, i, r.nb))) return rc;
         i += r.nb;
         *fed = i;
     }
@@ -1229,6 +1235,14 @@ int run_batch_step(axq_model *m, int max_pos_now) {
 template <class T>
 hipError_t dev_alloc(T **p, size_t count) { return hipMalloc((void **)p, (count ? count : 1) * sizeof(T)); }
 
+// After a failed call: back to position `base`, or to an empty sequence where the state cannot be rewound.
+void rewind_to(axq_model *m, int base) {
+    if (m->stack && axq_stack_recurrent(m)) base = 0;
+    set_i32_kernel<<<1, 1, 0, m->ctx->stream>>>(m->pos, base);
+    (void)hipStreamSynchronize(m->ctx->stream);
+    m->host_pos = base;
+}
+
 // The captured steps hold device addresses: whoever replaces a buffer they read drops them; the next step captures anew.
 void invalidate_graphs(axq_model *m) {
     if (m->graph_ok) (void)hipGraphExecDestroy(m->graph);
@@ -1239,6 +1253,32 @@ void invalidate_graphs(axq_model *m) {
 }
 
 } // namespace
+
+void axq_model_drop_graphs(axq_model *m) { invalidate_graphs(m); }
+
+int axq_model_alloc_common(axq_model *m) {
+    axq_ctx *ctx = m->ctx;
+    const axq_model_config &c = m->cfg;
+    const char *chunk = getenv("AXQ_PROMPT_CHUNK"); // development knob: fewer prompt rows per pass (tests cross chunk borders with it)
+    m->prompt_chunk = chunk ? atoi(chunk) : PROMPT_CHUNK;
+    if (m->prompt_chunk < PROMPT_GEMM_MIN) m->prompt_chunk = PROMPT_GEMM_MIN;
+    if (m->prompt_chunk > PROMPT_CHUNK) m->prompt_chunk = PROMPT_CHUNK;
+    m->n_seq = 1;
+    m->seq_pos.assign(1, 0);
+    m->prompt_cap = m->out_cap = c.max_position_embeddings;
+    hipError_t e = dev_alloc(&m->h, c.hidden_size);
+    if (e == hipSuccess) e = dev_alloc(&m->logits, c.vocab_size);
+    for (int32_t **p : {&m->pos, &m->tok, &m->next, &m->gen})
+        if (e == hipSuccess) e = dev_alloc(p, 1);
+    if (e == hipSuccess) e = dev_alloc(&m->prompt, m->prompt_cap);
+    if (e == hipSuccess) e = dev_alloc(&m->out, m->out_cap);
+    if (e == hipSuccess) e = dev_alloc(&m->hist, c.max_position_embeddings);
+    if (e == hipSuccess) e = hipMemsetAsync(m->pos, 0, 4, ctx->stream);
+    if (e == hipSuccess) e = hipMemsetAsync(m->gen, 0, 4, ctx->stream);
+    if (e == hipSuccess) e = hipMemsetAsync(m->tok, 0, 4, ctx->stream);
+    if (e != hipSuccess) return axq_fail(ctx, AXQ_ERR_ALLOCATION_FAILED, "model buffers: %s", hipGetErrorString(e));
+    return AXQ_OK;
+}
 
 extern "C" {
 
@@ -1278,20 +1318,17 @@ int axq_model_create(axq_ctx *ctx, const axq_model_config *cfg, axq_model **out)
         m->fused_max = knob ? atoi(knob) : 240;
         if (m->fused_max > 32768) m->fused_max = 32768;
         m->attn_mfma = !(getenv("AXQ_ATTN_MFMA") && getenv("AXQ_ATTN_MFMA")[0] == '0');
-        const char *chunk = getenv("AXQ_PROMPT_CHUNK"); // development knob: fewer prompt rows per pass (tests cross chunk borders with it)
-        m->prompt_chunk = chunk ? atoi(chunk) : PROMPT_CHUNK;
-        if (m->prompt_chunk < PROMPT_GEMM_MIN) m->prompt_chunk = PROMPT_GEMM_MIN;
-        if (m->prompt_chunk > PROMPT_CHUNK) m->prompt_chunk = PROMPT_CHUNK;
     }
-    m->n_seq = 1;
     m->seq_stride = (size_t)c.num_hidden_layers * c.num_key_value_heads * c.max_position_embeddings * c.head_dim;
-    m->seq_pos.assign(1, 0);
     const int L = c.num_hidden_layers, H = c.hidden_size, I = c.intermediate_size;
     m->w_qkv.assign(L, nullptr); m->w_o.assign(L, nullptr); m->w_gu.assign(L, nullptr); m->w_down.assign(L, nullptr);
     for (auto &v : m->w_sep) v.assign(L, nullptr);
     m->set_mask.assign(L, 0);
-    m->prompt_cap = c.max_position_embeddings;
-    m->out_cap = c.max_position_embeddings;
+    int rc0 = axq_model_alloc_common(m);
+    if (rc0) {
+        axq_model_free(m);
+        return rc0;
+    }
     const size_t kv = (size_t)L * c.num_key_value_heads * c.max_position_embeddings * c.head_dim;
     hipError_t e = hipSuccess;
 #define TRY(x) if (e == hipSuccess) e = (x)
@@ -1299,17 +1336,14 @@ int axq_model_create(axq_ctx *ctx, const axq_model_config *cfg, axq_model **out)
     TRY(dev_alloc(&m->rope_cos, (size_t)c.max_position_embeddings * c.head_dim / 2));
     TRY(dev_alloc(&m->rope_sin, (size_t)c.max_position_embeddings * c.head_dim / 2));
     TRY(dev_alloc(&m->kcache, kv)); TRY(dev_alloc(&m->vcache, kv));
-    TRY(dev_alloc(&m->h, H)); TRY(dev_alloc(&m->xn, H)); TRY(dev_alloc(&m->qkv, m->qkv_rows)); TRY(dev_alloc(&m->att, m->q_dim));
+    TRY(dev_alloc(&m->xn, H)); TRY(dev_alloc(&m->qkv, m->qkv_rows)); TRY(dev_alloc(&m->att, m->q_dim));
     m->part_stride = (size_t)c.num_key_value_heads * m->max_splits * (c.num_attention_heads / c.num_key_value_heads) * (c.head_dim + 2);
     TRY(dev_alloc(&m->att_part, m->part_stride));
-    TRY(dev_alloc(&m->gu, (size_t)2 * I)); TRY(dev_alloc(&m->act, I)); TRY(dev_alloc(&m->logits, c.vocab_size));
+    TRY(dev_alloc(&m->gu, (size_t)2 * I)); TRY(dev_alloc(&m->act, I));
     m->pb_cap = PROMPT_BATCH;
     TRY(dev_alloc(&m->pb_h, (size_t)PROMPT_BATCH * H)); TRY(dev_alloc(&m->pb_xn, (size_t)MAX_SEQUENCES * (H > I ? H : I))); // normalised rows in front of the lm_head and of linears outside the GEMV's reach
     TRY(dev_alloc(&m->pb_qkv, (size_t)PROMPT_BATCH * m->qkv_rows)); TRY(dev_alloc(&m->pb_att, (size_t)PROMPT_BATCH * m->q_dim));
     TRY(dev_alloc(&m->pb_gu, (size_t)PROMPT_BATCH * 2 * I)); TRY(dev_alloc(&m->pb_act, (size_t)PROMPT_BATCH * I));
-    TRY(dev_alloc(&m->pos, 1)); TRY(dev_alloc(&m->tok, 1)); TRY(dev_alloc(&m->next, 1)); TRY(dev_alloc(&m->gen, 1));
-    TRY(dev_alloc(&m->prompt, m->prompt_cap)); TRY(dev_alloc(&m->out, m->out_cap));
-    TRY(dev_alloc(&m->hist, c.max_position_embeddings));
 #undef TRY
     if (e != hipSuccess) {
         int rc = axq_fail(ctx, AXQ_ERR_ALLOCATION_FAILED, "model buffers: %s", hipGetErrorString(e));
@@ -1324,9 +1358,6 @@ int axq_model_create(axq_ctx *ctx, const axq_model_config *cfg, axq_model **out)
     {
         hipError_t e = hipMemsetAsync(m->kcache, 0, kv * 2, ctx->stream);
         if (e == hipSuccess) e = hipMemsetAsync(m->vcache, 0, kv * 2, ctx->stream);
-        if (e == hipSuccess) e = hipMemsetAsync(m->pos, 0, 4, ctx->stream);
-        if (e == hipSuccess) e = hipMemsetAsync(m->gen, 0, 4, ctx->stream);
-        if (e == hipSuccess) e = hipMemsetAsync(m->tok, 0, 4, ctx->stream);
         if (e != hipSuccess) {
             const int st = axq_fail(ctx, AXQ_ERR_DRIVER, "axq_model_create: clearing the cache and the counters: %s", hipGetErrorString(e));
             axq_model_free(m);
@@ -1362,6 +1393,7 @@ void axq_model_free(axq_model *m) {
     if (!m) return;
     axq_ctx *ctx = m->ctx;
     (void)hipStreamSynchronize(ctx->stream);
+    axq_stack_free(m);
     if (m->graph_ok) (void)hipGraphExecDestroy(m->graph);
     if (m->graph_f_ok) (void)hipGraphExecDestroy(m->graph_f);
     if (m->graph_b_ok) (void)hipGraphExecDestroy(m->graph_b);
@@ -1413,6 +1445,7 @@ int axq_model_set_embedding_f32(axq_model *m, const float *table, int mem) {
 int axq_model_set_norm(axq_model *m, int layer, int which, const float *w, int mem) {
     if (!m || !w) return AXQ_ERR_INVALID_ARGUMENT;
     axq_ctx *ctx = m->ctx;
+    if (m->stack) return axq_fail(ctx, AXQ_ERR_INVALID_ARGUMENT, "axq_model_set_norm: a model of described layers takes axq_model_set_tensor");
     const int H = m->cfg.hidden_size;
     if (layer >= m->cfg.num_hidden_layers || (layer >= 0 && (which < 0 || which > 1)))
         return axq_fail(ctx, AXQ_ERR_INVALID_ARGUMENT, "axq_model_set_norm: layer %d / which %d out of range", layer, which);
@@ -1426,6 +1459,7 @@ int axq_model_set_norm(axq_model *m, int layer, int which, const float *w, int m
 int axq_model_set_linear(axq_model *m, int layer, int which, const axq_weight *w) {
     if (!m || !w) return AXQ_ERR_INVALID_ARGUMENT;
     axq_ctx *ctx = m->ctx;
+    if (m->stack) return axq_fail(ctx, AXQ_ERR_INVALID_ARGUMENT, "axq_model_set_linear: a model of described layers takes axq_model_set_tensor");
     if (layer >= m->cfg.num_hidden_layers)
         return axq_fail(ctx, AXQ_ERR_INVALID_ARGUMENT, "axq_model_set_linear: layer %d out of range", layer);
     int64_t rows, k;
@@ -1499,6 +1533,7 @@ int axq_model_set_linear(axq_model *m, int layer, int which, const axq_weight *w
 int axq_model_random_init(axq_model *m, int type, float std, uint64_t seed) {
     if (!m) return AXQ_ERR_INVALID_ARGUMENT;
     axq_ctx *ctx = m->ctx;
+    if (m->stack) return axq_stack_random_init(m, std, seed);
     const axq_model_config &c = m->cfg;
     size_t max_elems = (size_t)c.vocab_size * c.hidden_size;
     for (int which = 0; which < AXQ_LIN_COUNT; which++) {
@@ -1554,6 +1589,9 @@ int axq_model_truncate(axq_model *m, int n_positions) {
     if (n_positions < 0 || n_positions > m->host_pos)
         return axq_fail(ctx, AXQ_ERR_INVALID_ARGUMENT, "axq_model_truncate: %d positions asked, the cache holds %d", n_positions,
                         m->host_pos);
+    if (m->stack && axq_stack_recurrent(m) && n_positions != 0 && n_positions != m->host_pos)
+        return axq_fail(ctx, AXQ_ERR_INVALID_ARGUMENT, "axq_model_truncate: a recurrent state of %d positions cannot be rewound to %d (only to 0)",
+                        m->host_pos, n_positions);
     set_i32_kernel<<<1, 1, 0, ctx->stream>>>(m->pos, n_positions);
     AXQ_HIP(ctx, hipStreamSynchronize(ctx->stream), AXQ_ERR_DRIVER);
     m->host_pos = n_positions;
@@ -1566,7 +1604,10 @@ int axq_model_set_batch(axq_model *m, int n_seq) {
     const axq_model_config &c = m->cfg;
     if (n_seq < 1 || n_seq > MAX_SEQUENCES)
         return axq_fail(ctx, AXQ_ERR_INVALID_ARGUMENT, "axq_model_set_batch: 1 to %d sequences, got %d", MAX_SEQUENCES, n_seq);
-
+    if (m->stack) {
+        if (n_seq > 1) return axq_fail(ctx, AXQ_ERR_SHAPE_MISMATCH, "Shape mismatch: a model of described layers holds one sequence");
+        return axq_model_reset(m);
+    }
     if (n_seq > 1 && (c.vocab_size % 4 != 0 || prompt_attn_lds(m, c.max_position_embeddings) > 128 * 1024))
         return axq_fail(ctx, AXQ_ERR_SHAPE_MISMATCH,
                         "Shape mismatch: batched steps need a vocabulary that is a multiple of 4 and at most 32768 positions "
@@ -1655,6 +1696,9 @@ int axq_model_forward_batch(axq_model *m, const int32_t *tokens, float *logits, 
     if (!m || !tokens) return AXQ_ERR_INVALID_ARGUMENT;
     axq_ctx *ctx = m->ctx;
     int rc;
+    if (m->stack) { // one sequence: its step
+        return axq_model_forward(m, tokens[0], logits, next_tokens);
+    }
     if ((rc = check_ready(m))) return rc;
     const int S = m->n_seq, V = m->cfg.vocab_size;
     m->seq_pos[0] = m->host_pos;
@@ -1685,6 +1729,11 @@ int axq_model_generate_batch(axq_model *m, const int32_t *prompts, const int32_t
     if (!m || !prompts || !offsets || !out_tokens) return AXQ_ERR_INVALID_ARGUMENT;
     axq_ctx *ctx = m->ctx;
     int rc;
+    if (m->stack) {
+        if (offsets[0] != 0) return axq_fail(ctx, AXQ_ERR_SHAPE_MISMATCH, "Shape mismatch: offsets start at 0");
+        if ((rc = axq_model_reset(m))) return rc;
+        return axq_model_generate(m, prompts, offsets[1], max_new_tokens, out_tokens, prefill_ms, decode_ms);
+    }
     if ((rc = check_ready(m))) return rc;
     const int S = m->n_seq, P = m->cfg.max_position_embeddings;
     if (max_new_tokens < 1 || max_new_tokens > m->out_cap || offsets[0] != 0)
@@ -1772,6 +1821,7 @@ int axq_model_seq_len(const axq_model *m) { return m ? m->host_pos : -1; }
 int axq_model_read_kv(axq_model *m, int layer, int which, uint16_t *out) {
     if (!m || !out || layer < 0 || layer >= m->cfg.num_hidden_layers) return AXQ_ERR_INVALID_ARGUMENT;
     axq_ctx *ctx = m->ctx;
+    if (m->stack) return axq_fail(ctx, AXQ_ERR_INVALID_ARGUMENT, "axq_model_read_kv: described layers keep no such cache");
     size_t per_layer = (size_t)m->cfg.num_key_value_heads * m->cfg.max_position_embeddings * m->cfg.head_dim;
     const uint16_t *src = (which ? m->vcache : m->kcache) + (size_t)layer * per_layer;
     AXQ_HIP(ctx, hipMemcpyAsync(out, src, per_layer * 2, hipMemcpyDeviceToHost, ctx->stream), AXQ_ERR_COPY_FAILED);
@@ -1827,8 +1877,7 @@ int axq_model_forward_tokens(axq_model *m, const int32_t *tokens, int n, float *
     AXQ_HIP(ctx, hipMemcpyAsync(m->prompt, tokens, (size_t)n * 4, hipMemcpyHostToDevice, ctx->stream), AXQ_ERR_COPY_FAILED);
     rc = feed_prompt(m, m->host_pos, n);
     if (rc) { // the device-side position may have moved: bring both sides back to where the call started
-        set_i32_kernel<<<1, 1, 0, ctx->stream>>>(m->pos, m->host_pos);
-        (void)hipStreamSynchronize(ctx->stream);
+        rewind_to(m, m->host_pos);
         return rc;
     }
     m->host_pos += n;
@@ -1838,6 +1887,39 @@ int axq_model_forward_tokens(axq_model *m, const int32_t *tokens, int n, float *
     if (next_token)
         AXQ_HIP(ctx, hipMemcpyAsync(next_token, m->next, 4, hipMemcpyDeviceToHost, ctx->stream), AXQ_ERR_COPY_FAILED);
     AXQ_HIP(ctx, hipStreamSynchronize(ctx->stream), AXQ_ERR_DRIVER);
+    return AXQ_OK;
+}
+
+int axq_model_layer_runs(const axq_model *m) { return !m ? -1 : (m->stack ? axq_stack_layer_runs(m) : m->cfg.num_hidden_layers); }
+
+int axq_model_forward_rows(axq_model *m, const int32_t *tokens, int n, const int32_t *want, int n_want, float *logits, float *layers) {
+    if (!m || !tokens || n_want < 0 || (n_want > 0 && (!want || !logits))) return AXQ_ERR_INVALID_ARGUMENT;
+    axq_ctx *ctx = m->ctx;
+    int rc;
+    if ((rc = check_ready(m))) return rc;
+    if (n <= 0) return axq_fail(ctx, AXQ_ERR_SHAPE_MISMATCH, "Shape mismatch: at least one token is needed");
+    if (m->host_pos + n > m->cfg.max_position_embeddings)
+        return axq_fail(ctx, AXQ_ERR_OVERFLOW, "Numerical overflow during quantization: %d + %d positions exceed the cache of %d",
+                        m->host_pos, n, m->cfg.max_position_embeddings);
+    for (int i = 0; i < n; i++)
+        if (tokens[i] < 0 || tokens[i] >= m->cfg.vocab_size)
+            return axq_fail(ctx, AXQ_ERR_INVALID_ARGUMENT, "token %d outside the vocabulary of %d", tokens[i], m->cfg.vocab_size);
+    for (int j = 0; j < n_want; j++)
+        if (want[j] < 0 || want[j] >= n || (j > 0 && want[j] <= want[j - 1]))
+            return axq_fail(ctx, AXQ_ERR_INVALID_ARGUMENT, "axq_model_forward_rows: places must rise within the %d tokens", n);
+    if (layers && !m->stack) return axq_fail(ctx, AXQ_ERR_INVALID_ARGUMENT, "axq_model_forward_rows: layer outputs are kept for described layers only");
+    AXQ_HIP(ctx, hipSetDevice(ctx->device), AXQ_ERR_DRIVER);
+    AXQ_HIP(ctx, hipMemcpyAsync(m->prompt, tokens, (size_t)n * 4, hipMemcpyHostToDevice, ctx->stream), AXQ_ERR_COPY_FAILED);
+    const Wanted w = {want, n_want, n, logits, layers};
+    int fed = 0;
+    rc = feed_rows(m, 0, m->prompt, n, m->host_pos, &fed, &w);
+    if (!rc && fed != n) rc = axq_fail(ctx, AXQ_ERR_SHAPE_MISMATCH, "Shape mismatch: the tokens cannot go through the layers as rows");
+    hipError_t e = hipStreamSynchronize(ctx->stream);
+    if (rc || e != hipSuccess) {
+        rewind_to(m, m->host_pos);
+        return rc ? rc : axq_fail(ctx, AXQ_ERR_DRIVER, "axq_model_forward_rows: %s", hipGetErrorString(e));
+    }
+    m->host_pos += n;
     return AXQ_OK;
 }
 
@@ -1882,8 +1964,7 @@ int axq_model_generate(axq_model *m, const int32_t *prompt, int n_prompt, int ma
     }
     (void)hipEventDestroy(e0); (void)hipEventDestroy(e1); (void)hipEventDestroy(e2);
     if (rc || e != hipSuccess) { // the device-side position may have moved: bring both sides back to where the call started
-        set_i32_kernel<<<1, 1, 0, ctx->stream>>>(m->pos, base);
-        (void)hipStreamSynchronize(ctx->stream);
+        rewind_to(m, base);
         return rc ? rc : axq_fail(ctx, AXQ_ERR_DRIVER, "generate: %s", hipGetErrorString(e));
     }
     m->host_pos = base + n_prompt + (max_new_tokens > 0 ? max_new_tokens - 1 : 0);

@@ -1,0 +1,520 @@
+// Products with bfloat16 weights: the GEMV of a decode step (input transforms, activations and residual adds ride in
+// it) and the GEMM of many rows (bf16 rows on the matrix pipe, or f32 rows in true 32-bit), both over several weights
+// per launch; and the row operations of a prompt around them.
+#include <hip/hip_bf16.h>
+
+#include "axq_dense.h"
+
+namespace {
+
+typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
+typedef float f32x16 __attribute__((ext_vector_type(16)));
+typedef uint32_t u32x4 __attribute__((ext_vector_type(4)));
+typedef const __attribute__((address_space(1))) void gbl_void;
+typedef __attribute__((address_space(3))) void lds_void;
+
+__device__ inline float tanh_norm(float x, float alpha, float w, float b) { return tanhf(alpha * x) * w + b; }
+
+// ---------------------------------------------------------------------------------------------------------------------
+// GEMV.  A workgroup stages f(x) in LDS once per distinct input and walks a contiguous range of row blocks (4 R rows,
+// R per wave); a lane's step is 16 bytes (8 weights) of each of its R rows.  x lies in LDS as two planes, elements
+// 8c .. 8c + 3 and 8c + 4 .. 8c + 7 of every chunk c, so that both 16-byte reads of a wave are free of bank conflicts.
+// ---------------------------------------------------------------------------------------------------------------------
+struct GemvArgs {
+    axq_parts parts;
+    axq_in in;
+    int steps; // of 512 elements
+};
+
+template <int MODE>
+__device__ void stage_x(const GemvArgs &a, const float *mu, float *xs, float *scratch) {
+    const axq_in &in = a.in;
+    const int k = in.k, tid = threadIdx.x, xl = a.steps * 512, half = xl >> 1;
+    auto slot = [half](int e) { return ((e >> 3) << 2) + (e & 3) + ((e & 4) ? half : 0); };
+    if (MODE == AXQ_IN_RMS_GATE) {
+        float ss = 0.f;
+        for (int e = tid; e < k; e += 256) {
+            const float v = in.x[e];
+            xs[slot(e)] = v;
+            ss = fmaf(v, v, ss);
+        }
+        ss = axq_block_sum(ss, scratch);
+        const float inv = 1.0f / sqrtf(ss / (float)k + in.eps);
+        for (int e = tid; e < xl; e += 256) xs[slot(e)] = e < k ? xs[slot(e)] * inv * in.nw[e] * in.gate[e] : 0.f;
+    } else if (MODE == AXQ_IN_POLY_NORM) {
+        float s1 = 0.f, s2 = 0.f, s3 = 0.f;
+        for (int e = tid; e < k; e += 256) {
+            const float z = in.x[e], z2 = z * z, z3 = z2 * z;
+            xs[slot(e)] = z;
+            s1 += z2; s2 = fmaf(z2, z2, s2); s3 = fmaf(z3, z3, s3);
+        }
+        s1 = axq_block_sum(s1, scratch);
+        s2 = axq_block_sum(s2, scratch);
+        s3 = axq_block_sum(s3, scratch);
+        const float c1 = in.coef[0] / sqrtf(s1 / (float)k + in.eps), c2 = in.coef[1] / sqrtf(s2 / (float)k + in.eps);
+        const float c3 = in.coef[2] / sqrtf(s3 / (float)k + in.eps), c0 = in.coef[3];
+        for (int e = tid; e < xl; e += 256) {
+            const float z = e < k ? xs[slot(e)] : 0.f;
+            xs[slot(e)] = e < k ? fmaf(fmaf(fmaf(c3, z, c2), z, c1), z, c0) : 0.f;
+        }
+    } else {
+        const float alpha = MODE == AXQ_IN_PLAIN ? 0.f : in.alpha[0];
+        const bool first = MODE == AXQ_IN_TANH_NORM_MIX && in.pos[0] == 0;
+        for (int e = tid; e < xl; e += 256) {
+            float v = 0.f;
+            if (e < k) {
+                v = in.x[e];
+                if (MODE != AXQ_IN_PLAIN) v = tanh_norm(v, alpha, in.nw[e], in.nb[e]);
+                if (MODE == AXQ_IN_TANH_NORM_MIX && mu) {
+                    const float p = first ? 0.f : in.prev[e];
+                    v = fmaf(p - v, mu[e], v);
+                }
+            }
+            xs[slot(e)] = v;
+        }
+    }
+    __syncthreads();
+}
+
+template <int MODE, int R>
+__global__ void __launch_bounds__(256) dense_gemv_kernel(GemvArgs a) {
+    extern __shared__ __attribute__((aligned(16))) float xs[];
+    __shared__ float scratch[16];
+    constexpr int U = 8 / R;
+    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+    const int nb = a.parts.n_blocks, b0 = (int)((long long)nb * blockIdx.x / gridDim.x), b1 = (int)((long long)nb * (blockIdx.x + 1) / gridDim.x);
+    const int half = a.steps * 256, k8 = (a.in.k + 7) >> 3;
+    int staged = -1;
+    for (int b = b0; b < b1; b++) {
+        int pi = 0;
+        while (pi + 1 < a.parts.n_parts && b >= a.parts.p[pi + 1].blk0) pi++;
+        const axq_part &p = a.parts.p[pi];
+        if (staged < 0 || (MODE == AXQ_IN_TANH_NORM_MIX && staged != pi)) {
+            if (staged >= 0) __syncthreads();
+            stage_x<MODE>(a, p.mu, xs, scratch);
+            staged = pi;
+        }
+        const int row0 = (b - p.blk0) * 4 * R + wave * R;
+        const uint16_t *w[R];
+        float acc[R];
+#pragma unroll
+        for (int r = 0; r < R; r++) {
+            const int row = row0 + r < p.n ? row0 + r : p.n - 1;
+            w[r] = p.w + (size_t)row * p.ldw;
+            acc[r] = 0.f;
+        }
+        for (int s0 = 0; s0 < a.steps; s0 += U) {
+            u32x4 q[U][R];
+#pragma unroll
+            for (int u = 0; u < U; u++) {
+                int c = (s0 + u) * 64 + lane; // past the row's end: a valid chunk against zeros
+                c = c < k8 ? c : k8 - 1;
+#pragma unroll
+                for (int r = 0; r < R; r++) q[u][r] = __builtin_nontemporal_load(reinterpret_cast<const u32x4 *>(w[r] + (size_t)c * 8));
+            }
+#pragma unroll
+            for (int u = 0; u < U; u++) {
+                if (s0 + u < a.steps) {
+                    const int c = (s0 + u) * 64 + lane;
+                    const float4 xa = *reinterpret_cast<const float4 *>(xs + c * 4), xb = *reinterpret_cast<const float4 *>(xs + half + c * 4);
+#pragma unroll
+                    for (int r = 0; r < R; r++) {
+                        float t = acc[r];
+                        t = fmaf(axq_bf16_lo(q[u][r][0]), xa.x, t); t = fmaf(axq_bf16_hi(q[u][r][0]), xa.y, t);
+                        t = fmaf(axq_bf16_lo(q[u][r][1]), xa.z, t); t = fmaf(axq_bf16_hi(q[u][r][1]), xa.w, t);
+                        t = fmaf(axq_bf16_lo(q[u][r][2]), xb.x, t); t = fmaf(axq_bf16_hi(q[u][r][2]), xb.y, t);
+                        t = fmaf(axq_bf16_lo(q[u][r][3]), xb.z, t); t = fmaf(axq_bf16_hi(q[u][r][3]), xb.w, t);
+                        acc[r] = t;
+                    }
+                }
+            }
+        }
+#pragma unroll
+        for (int r = 0; r < R; r++) acc[r] = axq_wave_sum(acc[r]);
+        float v = acc[0];
+#pragma unroll
+        for (int r = 1; r < R; r++) v = lane == r ? acc[r] : v;
+        const int row = row0 + lane;
+        if (lane < R && row < p.n) {
+            if (p.bias) v += p.bias[row];
+            v = axq_act(p.act, v, a.parts.cap);
+            p.y[row] = p.add ? p.y[row] + v : v;
+        }
+    }
+}
+
+template <int MODE, int R>
+int launch_gemv(axq_ctx *ctx, GemvArgs &a) {
+    int nb = 0;
+    for (int i = 0; i < a.parts.n_parts; i++) {
+        a.parts.p[i].blk0 = nb;
+        nb += (a.parts.p[i].n + 4 * R - 1) / (4 * R);
+    }
+    a.parts.n_blocks = nb;
+    const int most = 2 * ctx->prop.multiProcessorCount;
+    const size_t lds = (size_t)a.steps * 512 * sizeof(float);
+    static std::atomic<uint64_t> lds_allowed{0};
+    int rc;
+    if (lds > 48 * 1024 &&
+        (rc = axq_allow_lds(ctx, reinterpret_cast<const void *>(&dense_gemv_kernel<MODE, R>), lds_allowed, (size_t)AXQ_DENSE_MAX_K * 4)))
+        return rc;
+    dense_gemv_kernel<MODE, R><<<nb < most ? nb : most, 256, lds, ctx->stream>>>(a);
+    AXQ_LAUNCH_CHECK(ctx, "dense_gemv_kernel");
+    return AXQ_OK;
+}
+
+template <int MODE>
+int launch_gemv_mode(axq_ctx *ctx, GemvArgs &a) {
+    long long rows = 0;
+    for (int i = 0; i < a.parts.n_parts; i++) rows += a.parts.p[i].n;
+    if (rows >= 8192) return launch_gemv<MODE, 4>(ctx, a);
+    if (rows >= 4096) return launch_gemv<MODE, 2>(ctx, a);
+    return launch_gemv<MODE, 1>(ctx, a);
+}
+
+// ---------------------------------------------------------------------------------------------------------------------
+// GEMM on bf16 rows: tiles of BM x BN, K in steps of 64, operands straight from memory into LDS (16 bytes per lane,
+// two stages).  Row r of a tile is 128 bytes of LDS whose 16-byte pieces are exchanged by r & 7 (the loads take the
+// permuted source address, the destination being fixed), so that the operand reads of eight rows use all banks.
+// The product is taken as D[row of x][row of W]: a lane's accumulators are one output column.
+// ---------------------------------------------------------------------------------------------------------------------
+struct GemmArgs {
+    axq_parts parts;
+    int m, k, ldx, mt, tiles;
+};
+
+__device__ inline int acc_row(int r, int lane) { return 8 * (r >> 2) + 4 * (lane >> 5) + (r & 3); }
+
+// Tiles in an order that gives each XCD (workgroups go round them) a contiguous run; a run walks the row tiles of a
+// column tile first, so that a weight tile is read by one XCD's L2.
+__device__ inline int xcd_tile(int tiles) {
+    const int b = blockIdx.x, per = tiles >> 3, rest = tiles & 7, x = b & 7;
+    return x * per + (x < rest ? x : rest) + (b >> 3);
+}
+
+template <int BM, int BN>
+__global__ void __launch_bounds__(256) dense_gemm_kernel(GemmArgs a) {
+    constexpr int MT = BM / 64, NT = BN / 64;          // 32 x 32 tiles of a wave (2 x 2 waves)
+    constexpr int AL = BM / 32, BL = BN / 32;          // 16-byte loads per thread and step
+    __shared__ __attribute__((aligned(16))) uint16_t lds[2][(BM + BN) * 64];
+    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, wm = wave >> 1, wn = wave & 1;
+    const int tile = xcd_tile(a.tiles), ct = tile / a.mt, m0 = (tile - ct * a.mt) * BM;
+    int pi = 0;
+    while (pi + 1 < a.parts.n_parts && ct >= a.parts.p[pi + 1].blk0) pi++;
+    const axq_part &p = a.parts.p[pi];
+    const int n0 = (ct - p.blk0) * BN;
+    const uint16_t *x = reinterpret_cast<const uint16_t *>(p.x);
+
+    const uint16_t *ga[AL], *gb[BL];
+#pragma unroll
+    for (int i = 0; i < AL; i++) {
+        const int idx = (i * 4 + wave) * 64 + lane, r = idx >> 3, c = (idx & 7) ^ (r & 7);
+        const int row = m0 + r < a.m ? m0 + r : a.m - 1;
+        ga[i] = x + (size_t)row * a.ldx + c * 8;
+    }
+#pragma unroll
+    for (int i = 0; i < BL; i++) {
+        const int idx = (i * 4 + wave) * 64 + lane, r = idx >> 3, c = (idx & 7) ^ (r & 7);
+        const int row = n0 + r < p.n ? n0 + r : p.n - 1;
+        gb[i] = p.w + (size_t)row * p.ldw + c * 8;
+    }
+    auto fetch = [&](int stage, int kt) {
+        uint16_t *la = lds[stage], *lb = la + BM * 64;
+#pragma unroll
+        for (int i = 0; i < AL; i++)
+            __builtin_amdgcn_global_load_lds((gbl_void *)(ga[i] + kt * 64), (lds_void *)(la + (i * 4 + wave) * 512), 16, 0, 0);
+#pragma unroll
+        for (int i = 0; i < BL; i++)
+            __builtin_amdgcn_global_load_lds((gbl_void *)(gb[i] + kt * 64), (lds_void *)(lb + (i * 4 + wave) * 512), 16, 0, 0);
+    };
+    f32x16 acc[MT][NT];
+#pragma unroll
+    for (int i = 0; i < MT; i++)
+#pragma unroll
+        for (int j = 0; j < NT; j++)
+#pragma unroll
+            for (int r = 0; r < 16; r++) acc[i][j][r] = 0.f;
+
+    const int kts = a.k >> 6, li = lane & 31, lh = lane >> 5;
+    fetch(0, 0);
+    for (int kt = 0; kt < kts; kt++) {
+        asm volatile("s_waitcnt vmcnt(0)" ::: "memory"); // this step's tile is in LDS ...
+        __syncthreads();                                  // ... of every wave, and nobody reads the other stage any more
+        if (kt + 1 < kts) fetch((kt + 1) & 1, kt + 1);
+        const uint16_t *la = lds[kt & 1], *lb = la + BM * 64;
+#pragma unroll
+        for (int ks = 0; ks < 4; ks++) {
+            bf16x8 fa[MT], fb[NT];
+#pragma unroll
+            for (int i = 0; i < MT; i++) {
+                const int r = wm * (BM / 2) + i * 32 + li;
+                fa[i] = *reinterpret_cast<const bf16x8 *>(la + r * 64 + (((ks * 2 + lh) ^ (r & 7)) << 3));
+            }
+#pragma unroll
+            for (int j = 0; j < NT; j++) {
+                const int r = wn * (BN / 2) + j * 32 + li;
+                fb[j] = *reinterpret_cast<const bf16x8 *>(lb + r * 64 + (((ks * 2 + lh) ^ (r & 7)) << 3));
+            }
+#pragma unroll
+            for (int i = 0; i < MT; i++)
+#pragma unroll
+                for (int j = 0; j < NT; j++) acc[i][j] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(fa[i], fb[j], acc[i][j], 0, 0, 0);
+        }
+    }
+#pragma unroll
+    for (int j = 0; j < NT; j++) {
+        const int n = n0 + wn * (BN / 2) + j * 32 + li;
+        if (n >= p.n) continue;
+        const float bias = p.bias ? p.bias[n] : 0.f;
+#pragma unroll
+        for (int i = 0; i < MT; i++)
+#pragma unroll
+            for (int r = 0; r < 16; r++) {
+                const int m = m0 + wm * (BM / 2) + i * 32 + acc_row(r, lane);
+                if (m < a.m) {
+                    float *y = p.y + (size_t)m * p.ldy + n;
+                    const float v = axq_act(p.act, acc[i][j][r] + bias, a.parts.cap);
+                    *y = p.add ? *y + v : v;
+                }
+            }
+    }
+}
+
+// GEMM on f32 rows in true 32-bit: 64 x 64 tiles, 4 x 4 results per thread, K in steps of 16.
+__global__ void __launch_bounds__(256) dense_gemm_f32_kernel(GemmArgs a) {
+    __shared__ __attribute__((aligned(16))) float as[16][68], bs[16][68];
+    const int tid = threadIdx.x, tx = tid & 15, ty = tid >> 4;
+    const int tile = xcd_tile(a.tiles), ct = tile / a.mt, m0 = (tile - ct * a.mt) * 64;
+    int pi = 0;
+    while (pi + 1 < a.parts.n_parts && ct >= a.parts.p[pi + 1].blk0) pi++;
+    const axq_part &p = a.parts.p[pi];
+    const int n0 = (ct - p.blk0) * 64;
+    const float *x = reinterpret_cast<const float *>(p.x);
+    const int lr = tid >> 2, lc = (tid & 3) * 4; // this thread's four elements of a step: row lr, columns lc ..
+    const float *ga = x + (size_t)(m0 + lr < a.m ? m0 + lr : a.m - 1) * a.ldx + lc;
+    const uint16_t *gb = p.w + (size_t)(n0 + lr < p.n ? n0 + lr : p.n - 1) * p.ldw + lc;
+    float acc[4][4];
+#pragma unroll
+    for (int i = 0; i < 4; i++)
+#pragma unroll
+        for (int j = 0; j < 4; j++) acc[i][j] = 0.f;
+    for (int k = 0; k < a.k; k += 16) {
+        const float4 va = *reinterpret_cast<const float4 *>(ga + k);
+        const uint2 vb = *reinterpret_cast<const uint2 *>(gb + k);
+        __syncthreads();
+        as[lc][lr] = va.x; as[lc + 1][lr] = va.y; as[lc + 2][lr] = va.z; as[lc + 3][lr] = va.w;
+        bs[lc][lr] = axq_bf16_lo(vb.x); bs[lc + 1][lr] = axq_bf16_hi(vb.x); bs[lc + 2][lr] = axq_bf16_lo(vb.y); bs[lc + 3][lr] = axq_bf16_hi(vb.y);
+        __syncthreads();
+#pragma unroll
+        for (int kk = 0; kk < 16; kk++) {
+            const float4 fa = *reinterpret_cast<const float4 *>(&as[kk][ty * 4]), fb = *reinterpret_cast<const float4 *>(&bs[kk][tx * 4]);
+            const float av[4] = {fa.x, fa.y, fa.z, fa.w}, bv[4] = {fb.x, fb.y, fb.z, fb.w};
+#pragma unroll
+            for (int i = 0; i < 4; i++)
+#pragma unroll
+                for (int j = 0; j < 4; j++) acc[i][j] = fmaf(av[i], bv[j], acc[i][j]);
+        }
+    }
+#pragma unroll
+    for (int i = 0; i < 4; i++)
+#pragma unroll
+        for (int j = 0; j < 4; j++) {
+            const int m = m0 + ty * 4 + i, n = n0 + tx * 4 + j;
+            if (m < a.m && n < p.n) {
+                float *y = p.y + (size_t)m * p.ldy + n;
+                const float v = axq_act(p.act, acc[i][j] + (p.bias ? p.bias[n] : 0.f), a.parts.cap);
+                *y = p.add ? *y + v : v;
+            }
+        }
+}
+
+int count_tiles(GemmArgs &a, int bm, int bn) {
+    int ct = 0;
+    for (int i = 0; i < a.parts.n_parts; i++) {
+        a.parts.p[i].blk0 = ct;
+        ct += (a.parts.p[i].n + bn - 1) / bn;
+    }
+    a.parts.n_blocks = ct;
+    a.mt = (a.m + bm - 1) / bm;
+    return a.tiles = ct * a.mt;
+}
+
+// ---------------------------------------------------------------------------------------------------------------------
+// Row operations of a prompt, one workgroup per row.
+// ---------------------------------------------------------------------------------------------------------------------
+__device__ inline void put(const axq_rows_out &o, size_t row, int e, float v) {
+    if (o.f32) reinterpret_cast<float *>(o.x)[row * o.ldx + e] = v;
+    else reinterpret_cast<uint16_t *>(o.x)[row * o.ldx + e] = axq_to_bf16(v);
+}
+
+__global__ void __launch_bounds__(256) embed_pos_kernel(const uint16_t *emb16, const float *emb32, const float *pos_table, const int32_t *tok,
+                                                        const int32_t *pos, int pos0, int width, float *h) {
+    const int e = blockIdx.x * 256 + threadIdx.x, t = blockIdx.y;
+    if (e >= width) return;
+    const int p = pos ? pos[0] + t : pos0 + t;
+    const size_t i = (size_t)tok[t] * width + e;
+    const float v = emb32 ? emb32[i] : (float)__builtin_bit_cast(_Float16, emb16[i]);
+    h[(size_t)t * width + e] = pos_table ? v + pos_table[(size_t)p * width + e] : v;
+}
+
+struct MixPtrs { const float *mu[AXQ_MAX_PARTS]; };
+
+__global__ void __launch_bounds__(256) rows_tanh_norm_kernel(axq_in in, int m, int first, int n_mix, MixPtrs mix, axq_rows_out out) {
+    const int t = blockIdx.x;
+    const float alpha = in.alpha[0];
+    const float *h = in.x + (size_t)t * in.k;
+    for (int e = threadIdx.x; e < out.ldx; e += 256) {
+        const bool in_row = e < in.k;
+        const float nw = in_row ? in.nw[e] : 0.f, nb = in_row ? in.nb[e] : 0.f;
+        const float n = in_row ? tanh_norm(h[e], alpha, nw, nb) : 0.f;
+        if (n_mix == 0) {
+            put(out, t, e, n);
+            continue;
+        }
+        float p = 0.f;
+        if (in_row && t > 0) p = tanh_norm(h[e - in.k], alpha, nw, nb);
+        else if (in_row && !first) p = in.prev[e];
+        for (int i = 0; i < n_mix; i++) put(out, (size_t)i * m + t, e, in_row ? fmaf(p - n, mix.mu[i][e], n) : 0.f);
+    }
+}
+
+__global__ void __launch_bounds__(256) store_prev_kernel(axq_in in, int m, float *prev) {
+    const int e = blockIdx.x * 256 + threadIdx.x;
+    if (e < in.k) prev[e] = tanh_norm(in.x[(size_t)(m - 1) * in.k + e], in.alpha[0], in.nw[e], in.nb[e]);
+}
+
+// one workgroup per row and group (the last group's workgroup zeroes the tail)
+__global__ void __launch_bounds__(256) rows_rms_gate_kernel(axq_in in, int group, axq_rows_out out) {
+    __shared__ float scratch[16];
+    const int t = blockIdx.x, e0 = blockIdx.y * group;
+    const float *x = in.x + (size_t)t * in.k, *g = in.gate + (size_t)t * in.k;
+    float ss = 0.f;
+    for (int e = e0 + threadIdx.x; e < e0 + group; e += blockDim.x) ss = fmaf(x[e], x[e], ss);
+    ss = axq_block_sum(ss, scratch);
+    const float inv = 1.0f / sqrtf(ss / (float)group + in.eps);
+    for (int e = e0 + threadIdx.x; e < e0 + group; e += blockDim.x) put(out, t, e, x[e] * inv * in.nw[e] * g[e]);
+    if (blockIdx.y == gridDim.y - 1)
+        for (int e = in.k + threadIdx.x; e < out.ldx; e += blockDim.x) put(out, t, e, 0.f);
+}
+
+__global__ void __launch_bounds__(256) rows_poly_norm_kernel(axq_in in, axq_rows_out out) {
+    __shared__ float scratch[16];
+    const int t = blockIdx.x, k = in.k;
+    const float *x = in.x + (size_t)t * k;
+    float s1 = 0.f, s2 = 0.f, s3 = 0.f;
+    for (int e = threadIdx.x; e < k; e += 256) {
+        const float z = x[e], z2 = z * z, z3 = z2 * z;
+        s1 += z2; s2 = fmaf(z2, z2, s2); s3 = fmaf(z3, z3, s3);
+    }
+    s1 = axq_block_sum(s1, scratch);
+    s2 = axq_block_sum(s2, scratch);
+    s3 = axq_block_sum(s3, scratch);
+    const float c1 = in.coef[0] / sqrtf(s1 / (float)k + in.eps), c2 = in.coef[1] / sqrtf(s2 / (float)k + in.eps);
+    const float c3 = in.coef[2] / sqrtf(s3 / (float)k + in.eps), c0 = in.coef[3];
+    for (int e = threadIdx.x; e < out.ldx; e += 256) {
+        const float z = e < k ? x[e] : 0.f;
+        put(out, t, e, e < k ? fmaf(fmaf(fmaf(c3, z, c2), z, c1), z, c0) : 0.f);
+    }
+}
+
+__global__ void __launch_bounds__(64) rows_zero_tail_kernel(int k, axq_rows_out out) {
+    for (int e = k + threadIdx.x; e < out.ldx; e += 64) put(out, blockIdx.x, e, 0.f);
+}
+
+} // namespace
+
+int axq_dense_gemv(axq_ctx *ctx, int mode, const axq_in &in, axq_parts &parts) {
+    if (in.k < 1 || in.k > AXQ_DENSE_MAX_K || parts.n_parts < 1 || parts.n_parts > AXQ_MAX_PARTS)
+        return axq_fail(ctx, AXQ_ERR_SHAPE_MISMATCH, "Shape mismatch: a decode product takes 1 to %d inputs and 1 to %d weights, got %d and %d",
+                        AXQ_DENSE_MAX_K, AXQ_MAX_PARTS, in.k, parts.n_parts);
+    GemvArgs a;
+    a.parts = parts;
+    a.in = in;
+    a.steps = (in.k + 511) / 512;
+    switch (mode) {
+    case AXQ_IN_PLAIN: return launch_gemv_mode<AXQ_IN_PLAIN>(ctx, a);
+    case AXQ_IN_TANH_NORM: return launch_gemv_mode<AXQ_IN_TANH_NORM>(ctx, a);
+    case AXQ_IN_TANH_NORM_MIX: return launch_gemv_mode<AXQ_IN_TANH_NORM_MIX>(ctx, a);
+    case AXQ_IN_RMS_GATE: return launch_gemv_mode<AXQ_IN_RMS_GATE>(ctx, a);
+    case AXQ_IN_POLY_NORM: return launch_gemv_mode<AXQ_IN_POLY_NORM>(ctx, a);
+    default: return axq_fail(ctx, AXQ_ERR_INVALID_ARGUMENT, "axq_dense_gemv: unknown input mode %d", mode);
+    }
+}
+
+int axq_dev_dense_gemv(axq_ctx *ctx, const axq_weight *w, const float *x, const float *bias, float *y) {
+    axq_in in;
+    in.x = x;
+    in.k = (int)w->k;
+    axq_parts parts = {};
+    parts.n_parts = 1;
+    parts.p[0].w = reinterpret_cast<const uint16_t *>(w->codes);
+    parts.p[0].ldw = (int)(w->codes_pitch / 2);
+    parts.p[0].n = (int)w->n_rows;
+    parts.p[0].bias = bias;
+    parts.p[0].y = y;
+    return axq_dense_gemv(ctx, AXQ_IN_PLAIN, in, parts);
+}
+
+int axq_dense_gemm(axq_ctx *ctx, axq_parts &parts, int m, int k, int ldx, bool f32) {
+    GemmArgs a;
+    a.parts = parts;
+    a.m = m;
+    a.k = (k + 63) / 64 * 64;
+    a.ldx = ldx;
+    if (m < 1 || k < 1 || ldx % 64 != 0 || ldx < a.k || parts.n_parts < 1 || parts.n_parts > AXQ_MAX_PARTS)
+        return axq_fail(ctx, AXQ_ERR_SHAPE_MISMATCH, "Shape mismatch: %d rows of %d elements (%d apart), %d weights", m, k, ldx, parts.n_parts);
+    for (int i = 0; i < parts.n_parts; i++)
+        if (parts.p[i].ldw < a.k || parts.p[i].n < 1)
+            return axq_fail(ctx, AXQ_ERR_SHAPE_MISMATCH, "Shape mismatch: weight %d has rows of %d elements, %d wanted", i, parts.p[i].ldw, a.k);
+    if (f32) {
+        count_tiles(a, 64, 64);
+        dense_gemm_f32_kernel<<<a.tiles, 256, 0, ctx->stream>>>(a);
+    } else if (m > 64 && count_tiles(a, 128, 128) >= ctx->prop.multiProcessorCount) {
+        dense_gemm_kernel<128, 128><<<a.tiles, 256, 0, ctx->stream>>>(a);
+    } else {
+        count_tiles(a, 64, 64);
+        dense_gemm_kernel<64, 64><<<a.tiles, 256, 0, ctx->stream>>>(a);
+    }
+    AXQ_LAUNCH_CHECK(ctx, "dense_gemm_kernel");
+    return AXQ_OK;
+}
+
+int axq_rows_embed(axq_ctx *ctx, const uint16_t *emb16, const float *emb32, const float *pos_table, const int32_t *tok, const int32_t *pos,
+                   int pos0, int m, int width, float *h) {
+    embed_pos_kernel<<<dim3((width + 255) / 256, m), 256, 0, ctx->stream>>>(emb16, emb32, pos_table, tok, pos, pos0, width, h);
+    AXQ_LAUNCH_CHECK(ctx, "embed_pos_kernel");
+    return AXQ_OK;
+}
+
+int axq_rows_tanh_norm(axq_ctx *ctx, const axq_in &in, int m, bool first, int n_mix, const float *const *mu, axq_rows_out out) {
+    MixPtrs mix = {};
+    for (int i = 0; i < n_mix; i++) mix.mu[i] = mu[i];
+    rows_tanh_norm_kernel<<<m, 256, 0, ctx->stream>>>(in, m, first ? 1 : 0, n_mix, mix, out);
+    AXQ_LAUNCH_CHECK(ctx, "rows_tanh_norm_kernel");
+    return AXQ_OK;
+}
+
+int axq_store_prev(axq_ctx *ctx, const axq_in &in, int m, float *prev) {
+    store_prev_kernel<<<(in.k + 255) / 256, 256, 0, ctx->stream>>>(in, m, prev);
+    AXQ_LAUNCH_CHECK(ctx, "store_prev_kernel");
+    return AXQ_OK;
+}
+
+int axq_rows_rms_gate(axq_ctx *ctx, const axq_in &in, int m, int group, axq_rows_out out) {
+    rows_rms_gate_kernel<<<dim3(m, in.k / group), group <= 128 ? 64 : 256, 0, ctx->stream>>>(in, group, out);
+    AXQ_LAUNCH_CHECK(ctx, "rows_rms_gate_kernel");
+    return AXQ_OK;
+}
+
+int axq_rows_poly_norm(axq_ctx *ctx, const axq_in &in, int m, axq_rows_out out) {
+    rows_poly_norm_kernel<<<m, 256, 0, ctx->stream>>>(in, out);
+    AXQ_LAUNCH_CHECK(ctx, "rows_poly_norm_kernel");
+    return AXQ_OK;
+}
+
+int axq_rows_zero_tail(axq_ctx *ctx, int m, int k, axq_rows_out out) {
+    if (k == out.ldx) return AXQ_OK;
+    rows_zero_tail_kernel<<<m, 64, 0, ctx->stream>>>(k, out);
+    AXQ_LAUNCH_CHECK(ctx, "rows_zero_tail_kernel");
+    return AXQ_OK;
+}

@@ -313,6 +313,28 @@ struct GF16 {
     }
 };
 
+struct GBF16 { // rows are padded to a multiple of 64 elements
+    static constexpr bool PRESCALED = false;
+    static constexpr float WS = 1.0f;
+    struct Raw { uint4 v0, v1; };
+    __device__ static void load16(const GemmArgs &a, size_t row, int kstep, int u4, Raw &r) {
+        const uint4 *p = reinterpret_cast<const uint4 *>(a.codes + row * a.codes_pitch + ((size_t)kstep * 64 + u4 * 16) * 2);
+        r.v0 = p[0];
+        r.v1 = p[1];
+    }
+    __device__ static void cvt16(const Raw &r, int, int u4, float (&w)[16], int &k0, int &k1) {
+        const uint4 v0 = r.v0, v1 = r.v1;
+        const uint32_t qq[8] = {v0.x, v0.y, v0.z, v0.w, v1.x, v1.y, v1.z, v1.w};
+#pragma unroll
+        for (int i = 0; i < 8; i++) {
+            w[2 * i] = __builtin_bit_cast(float, qq[i] << 16);
+            w[2 * i + 1] = __builtin_bit_cast(float, qq[i] & 0xFFFF0000u);
+        }
+        k0 = u4 * 16;
+        k1 = k0 + 8;
+    }
+};
+
 struct GF32 {
     static constexpr bool PRESCALED = false;
     static constexpr float WS = 1.0f; // plain weights may be large: no headroom to give away
@@ -1694,6 +1716,7 @@ int run_gemm(axq_ctx *ctx, const axq_weight *w, int m, const GemmPlan &p, float 
     case AXQ_Q8_0: return launch_gemm<GQ80>(ctx, a, p.splits);
     case AXQ_F16: return launch_gemm<GF16>(ctx, a, p.splits);
     case AXQ_F32: return launch_gemm<GF32>(ctx, a, p.splits);
+    case AXQ_BF16: return launch_gemm<GBF16>(ctx, a, p.splits);
     default: return axq_fail(ctx, AXQ_ERR_INVALID_QUANT_TYPE, "Invalid quantization type: %d", w->type);
     }
 }

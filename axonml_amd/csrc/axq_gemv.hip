@@ -697,6 +697,7 @@ int axq_dev_gemv(axq_ctx *ctx, const axq_weight *w, const float *x, int batch, c
         if (rc < 0) return rc;
         if (rc == 1) continue;
         switch (w->type) {
+        case AXQ_BF16: rc = axq_dev_dense_gemv(ctx, w, xb, bias, yb); break;
         case AXQ_Q4_K: rc = launch<Q4K>(ctx, w, xb, bias, yb); break;
         case AXQ_Q6_K: rc = launch<Q6K>(ctx, w, xb, bias, yb); break;
         case AXQ_Q5_K: rc = launch<Q5K>(ctx, w, xb, bias, yb); break;

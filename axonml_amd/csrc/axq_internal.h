@@ -120,6 +120,8 @@ int axq_dev_repack(axq_ctx *ctx, const axq_weight *w, uint8_t *packed_dev, bool 
 int axq_weight_alloc(axq_ctx *ctx, int type, int64_t n_rows, int64_t k, axq_weight **out);
 // gemv.hip
 int axq_dev_gemv(axq_ctx *ctx, const axq_weight *w, const float *x_dev, int batch, const float *bias_dev, float *y_dev);
+// dense.hip: y = x W^T (+ bias) for one f32 vector and an AXQ_BF16 weight
+int axq_dev_dense_gemv(axq_ctx *ctx, const axq_weight *w, const float *x, const float *bias, float *y);
 // gemv_mfma.hip: 1 = launched, 0 = shape not covered, <0 = error
 int axq_dev_gemv_dp(axq_ctx *ctx, const axq_weight *w, const float *x, const uint8_t *xq, const float *bias, float *y);
 // What the GEMV does to x before it uses it (xq must be NULL for the fused forms):

@@ -69,6 +69,7 @@ int axq_weight_alloc(axq_ctx *ctx, int type, int64_t n_rows, int64_t k, axq_weig
     case AXQ_Q5_K: w->codes_pitch = (size_t)k / 2; meta_per_block = 16; qh_per_block = 32; break; // Q4_K's planes and the fifth bits as they are
     case AXQ_F16: w->codes_pitch = (size_t)k * 2; break;
     case AXQ_F32: w->codes_pitch = (size_t)k * 4; break;
+    case AXQ_BF16: w->codes_pitch = axq_align_up((size_t)k * 2, 128); break;
     }
     w->meta_pitch = type == AXQ_Q6_K ? axq_align_up(nblk * meta_per_block, 16) : nblk * meta_per_block;
     w->qh_pitch = nblk * qh_per_block;

@@ -1,6 +1,6 @@
 """Host-side mirror of the reference's LLaMA/Mistral decode loop over the axq C ABI.
 
-`QuantizedLlama` plays the part of LLaMAForCausalLM (crates/axonml-llm/src/llama.rs:834-1100) for one
+`QuantizedLlama` (a `DecoderModel`) plays the part of LLaMAForCausalLM (crates/axonml-llm/src/llama.rs:834-1100) for one
 sequence: `forward_with_cache`-style single-token steps and greedy `generate`, with every linear a
 quantized, device-resident weight.  Config field names follow LLaMAConfig / MistralConfig.
 """
@@ -22,49 +22,27 @@ def mistral_7b_config(max_position_embeddings=640):
                 max_position_embeddings=max_position_embeddings, rms_norm_eps=1e-5, rope_theta=10000.0, sliding_window=4096)
 
 
-class QuantizedLlama:
-    def __init__(self, ctx=None, **cfg):
-        self.ctx = ctx or default_context()
-        self.cfg = _lib.ModelConfig(**cfg)
-        h = C.c_void_p()
-        self.ctx.check(self.ctx.lib.axq_model_create(self.ctx.handle, C.byref(self.cfg), C.byref(h)))
-        self.handle = h
+class DecoderModel:
+    """What every decode model offers, whatever its layers are: an axq_model handle, its embedding, its steps, its generation
+    and its sampling.  A subclass creates the handle and loads the layers' weights."""
 
-    # ---- weights
+    def __init__(self, ctx, handle, vocab_size, hidden_size):
+        self.ctx, self.handle, self.vocab_size, self.hidden_size = ctx, handle, int(vocab_size), int(hidden_size)
+
     def set_embedding_f16(self, table_bits):
         t = np.ascontiguousarray(table_bits, dtype=np.uint16)
-        if t.size != self.cfg.vocab_size * self.cfg.hidden_size:
+        if t.size != self.vocab_size * self.hidden_size:
             raise ShapeMismatch(f"Shape mismatch: embedding table of {t.size} elements, expected vocab_size * hidden_size = "
-                                f"{self.cfg.vocab_size} * {self.cfg.hidden_size}")
+                                f"{self.vocab_size} * {self.hidden_size}")
         self.ctx.check(self.ctx.lib.axq_model_set_embedding_f16(self.handle, t.ctypes.data, MEM_HOST))
 
     def set_embedding_f32(self, table):
         """The embedding table in f32, as the reference keeps it (embedding.rs:103-146)."""
         t = np.ascontiguousarray(table, dtype=np.float32)
-        if t.size != self.cfg.vocab_size * self.cfg.hidden_size:
+        if t.size != self.vocab_size * self.hidden_size:
             raise ShapeMismatch(f"Shape mismatch: embedding table of {t.size} elements, expected vocab_size * hidden_size = "
-                                f"{self.cfg.vocab_size} * {self.cfg.hidden_size}")
+                                f"{self.vocab_size} * {self.hidden_size}")
         self.ctx.check(self.ctx.lib.axq_model_set_embedding_f32(self.handle, t.ctypes.data, MEM_HOST))
-
-    def set_norm(self, layer, which, w):
-        w = np.ascontiguousarray(w, dtype=np.float32)
-        if w.size != self.cfg.hidden_size:  # the library copies hidden_size floats from this pointer
-            raise ShapeMismatch(f"Shape mismatch: norm weight of {w.size} elements, expected hidden_size = {self.cfg.hidden_size}")
-        self.ctx.check(self.ctx.lib.axq_model_set_norm(self.handle, layer, which, w.ctypes.data, MEM_HOST))
-
-    def set_linear(self, layer, name, weight):
-        """weight: QuantizedTensor or DeviceWeight of the linear's [out, in] shape; layer -1 = lm_head."""
-        if name not in LINEARS:
-            raise KeyError(f"unknown linear {name!r}: one of {sorted(LINEARS)}")
-        dw = weight if isinstance(weight, DeviceWeight) else DeviceWeight.upload(weight, self.ctx)
-        try:
-            self.ctx.check(self.ctx.lib.axq_model_set_linear(self.handle, layer, LINEARS[name], dw.handle))
-        finally:
-            if dw is not weight:
-                dw.free()
-
-    def random_init(self, quant_type=QuantType.Q4_K, std=0.02, seed=1):
-        self.ctx.check(self.ctx.lib.axq_model_random_init(self.handle, int(quant_type), std, seed))
 
     def set_sampling(self, config=None, seed=0):
         """Next tokens by a GenerationConfig (temperature, top-k, top-p, repetition penalty over every token fed so
@@ -80,7 +58,7 @@ class QuantizedLlama:
         return self.ctx.lib.axq_model_seq_len(self.handle)
 
     def forward(self, token, want_logits=True):
-        logits = np.empty(self.cfg.vocab_size, dtype=np.float32) if want_logits else None
+        logits = np.empty(self.vocab_size, dtype=np.float32) if want_logits else None
         nxt = C.c_int32()
         self.ctx.check(self.ctx.lib.axq_model_forward(self.handle, int(token), logits.ctypes.data if want_logits else None,
                                                       C.byref(nxt)))
@@ -89,11 +67,29 @@ class QuantizedLlama:
     def forward_tokens(self, tokens, want_logits=True):
         """forward_with_cache on several tokens (a prompt): the last position's next token and logits."""
         t = np.ascontiguousarray(tokens, dtype=np.int32)
-        logits = np.empty(self.cfg.vocab_size, dtype=np.float32) if want_logits else None
+        logits = np.empty(self.vocab_size, dtype=np.float32) if want_logits else None
         nxt = C.c_int32()
         self.ctx.check(self.ctx.lib.axq_model_forward_tokens(self.handle, t.ctypes.data, t.size,
                                                              logits.ctypes.data if want_logits else None, C.byref(nxt)))
         return nxt.value, logits
+
+    def forward_rows(self, tokens, want=(), layers=False):
+        """A portion of a prompt as rows: the logits at the (rising) places `want` of `tokens` [len(want), vocab], and with
+        `layers` also the residual stream after every layer run [runs, len(tokens), hidden]."""
+        t = np.ascontiguousarray(tokens, dtype=np.int32).reshape(-1)
+        w = np.ascontiguousarray(want, dtype=np.int32).reshape(-1)
+        logits = np.empty((w.size, self.vocab_size), dtype=np.float32)
+        trace = np.empty((self.ctx.lib.axq_model_layer_runs(self.handle), t.size, self.hidden_size), dtype=np.float32) if layers else None
+        self.ctx.check(self.ctx.lib.axq_model_forward_rows(self.handle, t.ctypes.data, t.size, w.ctypes.data, w.size, logits.ctypes.data,
+                                                           trace.ctypes.data if layers else None))
+        return (logits, trace) if layers else logits
+
+    def feed(self, tokens, want=()):
+        """The next tokens of the sequence, one by the decode step, several as rows; the logits at the places `want`."""
+        if len(tokens) != 1:
+            return self.forward_rows(tokens, want)
+        _, logits = self.forward(tokens[0], want_logits=len(want) > 0)
+        return logits.reshape(1, -1) if len(want) else np.empty((0, self.vocab_size), dtype=np.float32)
 
     def set_batch(self, n_seq):
         """Caches and positions for n_seq sequences side by side (1..64); starts all of them afresh."""
@@ -115,7 +111,7 @@ class QuantizedLlama:
         t = np.ascontiguousarray(tokens, dtype=np.int32)
         if t.shape != (n,):
             raise ValueError(f"{n} tokens wanted, one per sequence")
-        logits = np.empty((n, self.cfg.vocab_size), dtype=np.float32) if want_logits else None
+        logits = np.empty((n, self.vocab_size), dtype=np.float32) if want_logits else None
         nxt = np.empty(n, dtype=np.int32)
         self.ctx.check(self.ctx.lib.axq_model_forward_batch(self.handle, t.ctypes.data, logits.ctypes.data if want_logits else None,
                                                             nxt.ctypes.data))
@@ -140,14 +136,8 @@ class QuantizedLlama:
         self.ctx.check(self.ctx.lib.axq_model_truncate(self.handle, int(n_positions)))
 
     def hidden(self):
-        out = np.empty(self.cfg.hidden_size, dtype=np.float32)
+        out = np.empty(self.hidden_size, dtype=np.float32)
         self.ctx.check(self.ctx.lib.axq_model_read_hidden(self.handle, out.ctypes.data))
-        return out
-
-    def kv(self, layer, which):
-        c = self.cfg
-        out = np.empty((c.num_key_value_heads, c.max_position_embeddings, c.head_dim), dtype=np.uint16)
-        self.ctx.check(self.ctx.lib.axq_model_read_kv(self.handle, layer, which, out.ctypes.data))
         return out
 
     def generate(self, prompt, max_new_tokens):
@@ -168,6 +158,42 @@ class QuantizedLlama:
             self.close()
         except Exception:
             pass
+
+
+class QuantizedLlama(DecoderModel):
+    def __init__(self, ctx=None, **cfg):
+        self.ctx = ctx or default_context()
+        self.cfg = _lib.ModelConfig(**cfg)
+        h = C.c_void_p()
+        self.ctx.check(self.ctx.lib.axq_model_create(self.ctx.handle, C.byref(self.cfg), C.byref(h)))
+        super().__init__(self.ctx, h, self.cfg.vocab_size, self.cfg.hidden_size)
+
+    # ---- weights
+    def set_norm(self, layer, which, w):
+        w = np.ascontiguousarray(w, dtype=np.float32)
+        if w.size != self.cfg.hidden_size:  # the library copies hidden_size floats from this pointer
+            raise ShapeMismatch(f"Shape mismatch: norm weight of {w.size} elements, expected hidden_size = {self.cfg.hidden_size}")
+        self.ctx.check(self.ctx.lib.axq_model_set_norm(self.handle, layer, which, w.ctypes.data, MEM_HOST))
+
+    def set_linear(self, layer, name, weight):
+        """weight: QuantizedTensor or DeviceWeight of the linear's [out, in] shape; layer -1 = lm_head."""
+        if name not in LINEARS:
+            raise KeyError(f"unknown linear {name!r}: one of {sorted(LINEARS)}")
+        dw = weight if isinstance(weight, DeviceWeight) else DeviceWeight.upload(weight, self.ctx)
+        try:
+            self.ctx.check(self.ctx.lib.axq_model_set_linear(self.handle, layer, LINEARS[name], dw.handle))
+        finally:
+            if dw is not weight:
+                dw.free()
+
+    def random_init(self, quant_type=QuantType.Q4_K, std=0.02, seed=1):
+        self.ctx.check(self.ctx.lib.axq_model_random_init(self.handle, int(quant_type), std, seed))
+
+    def kv(self, layer, which):
+        c = self.cfg
+        out = np.empty((c.num_key_value_heads, c.max_position_embeddings, c.head_dim), dtype=np.uint16)
+        self.ctx.check(self.ctx.lib.axq_model_read_kv(self.handle, layer, which, out.ctypes.data))
+        return out
 
 
 def _bench_q4_k_m_mix(ctx, m, cfg, prompt, new_tokens, weight_elems, mean_ctx, log):

@@ -137,6 +137,10 @@ class HFLoader:
     def has(self, name):
         return name in self._where
 
+    def shape(self, name):
+        """A tensor's shape, or None."""
+        return list(self._where[name].entries[name][1]) if name in self._where else None
+
     def get_tensor(self, name):
         if name not in self._where:
             raise WeightNotFound(name)

@@ -48,7 +48,9 @@ typedef struct axq_model axq_model;
  * the 256-element GGUF superblock types appended: Q4_K (144 bytes) and Q6_K (210 bytes: 128 bytes of low nibbles,
  * 64 of high bit pairs, sixteen int8 scales of 16 elements each, f16 d; w = d * scale * (q - 32)), the type llama.cpp
  * keeps output.weight and part of the value and down projections in when it writes "Q4_0" and "Q4_K_M" files; and
- * Q5_K (176 bytes: Q4_K's header, 32 bytes of fifth bits, 128 of low nibbles; w = d * sc * q - dmin * m, q in 0..31). */
+ * Q5_K (176 bytes: Q4_K's header, 32 bytes of fifth bits, 128 of low nibbles; w = d * sc * q - dmin * m, q in 0..31).
+ * BF16 (bfloat16, rounded to nearest even) is the type of checkpoints that are kept as they are: one element per block,
+ * like F16; on the device its rows are padded with zeros to a multiple of 64 elements. */
 typedef enum {
     AXQ_Q8_0 = 0,
     AXQ_Q4_0 = 1,
@@ -60,7 +62,8 @@ typedef enum {
     AXQ_Q4_K = 7,
     AXQ_Q6_K = 8,
     AXQ_Q5_K = 9,
-    AXQ_TYPE_COUNT = 10
+    AXQ_BF16 = 10,
+    AXQ_TYPE_COUNT = 11
 } axq_type;
 
 typedef enum {
@@ -236,6 +239,12 @@ AXQ_API int axq_model_forward(axq_model *m, int32_t token, float *logits, int32_
  * multiple of 256 up to 16384, else one by one; results agree with n calls of axq_model_forward to
  * rounding (sums are taken in another order). */
 AXQ_API int axq_model_forward_tokens(axq_model *m, const int32_t *tokens, int n, float *logits, int32_t *next_token);
+/* The same for a portion of a prompt whose logits are wanted at chosen places: `want` holds n_want rising indices into
+ * `tokens`, logits (host) becomes f32[n_want, vocab].  Every token goes through the layers as a row.  layers (host, may be
+ * NULL; models of described layers only): the residual stream after every layer run, f32[axq_model_layer_runs, n, hidden]. */
+AXQ_API int axq_model_forward_rows(axq_model *m, const int32_t *tokens, int n, const int32_t *want, int n_want, float *logits,
+                                   float *layers);
+AXQ_API int axq_model_layer_runs(const axq_model *m);
 /* Several sequences side by side (the batch dimension of forward_with_cache's input ids and of KVCache,
  * llama.rs:731-762, attention.rs:28-35): n_seq = 1..64 caches and position counters; a batched step feeds
  * one token of every sequence and reads the weights once for all of them (up to eight sequences through the
@@ -267,6 +276,49 @@ AXQ_API int axq_model_seq_len(const axq_model *m);
 AXQ_API int axq_model_read_hidden(axq_model *m, float *hidden_out);
 /* One layer's f16 cache, [kv_heads][max_position_embeddings][head_dim] (host); which 0 = keys, 1 = values. */
 AXQ_API int axq_model_read_kv(axq_model *m, int layer, int which, uint16_t *out);
+
+/* ---- models of described layers.  A design whose layers differ from each other is a list of layer descriptions; the
+ *      model made from it is an axq_model like the one above: the same calls step it, generate with it, sample for it,
+ *      count its positions and free it.  It holds one sequence.  Its layers keep a KV cache (attention) or a recurrent
+ *      state in f32 (the other mixers); a recurrent state cannot be rewound, so axq_model_truncate takes 0 or the current
+ *      length only, and a call that fails midway empties the sequence. ------------------------------------------------- */
+typedef enum {
+    AXQ_MIX_ATTENTION = 0, /* causal attention, weights sigmoid(score + a number per head), not normalised over the keys;
+                              per-head RMS norms on q and k; q times 1 + q_temp_coef ln(floor((p + 1) / q_temp_every) + 1);
+                              score = q.k * scale + learned bias by distance (bias_rows buckets up to bias_max) */
+    AXQ_MIX_LIGHTNING = 1, /* linear attention: S <- decay S + k v^T, o = S^T q; SiLU on q, k, v; gated RMS norm over all heads */
+    AXQ_MIX_WKV = 2        /* time mixing: inputs leaning to the previous token's, a decay per token, head and key channel
+                              (through decay_rank), a bonus for the current token, gated RMS norm per head */
+} axq_mixer;
+/* Norms are tanh(alpha x) w + b.  Feed-forward (ff > 0): W_down act(W_up n(x)), act(z) = a N(z) + b N(z^2) + c N(z^3) + e with
+ * N(z) = z / sqrt(mean(z^2) + eps). */
+typedef struct {
+    int32_t mixer;                          /* axq_mixer */
+    int32_t heads, kv_heads, dim, vdim;     /* kv_heads: attention only; wkv: vdim = dim */
+    int32_t ff;                             /* 0: no feed-forward sublayer */
+    int32_t bias_rows, bias_max;            /* attention; bias_rows 0: no distance bias */
+    int32_t q_temp_every;                   /* attention; 0: no query factor */
+    float q_temp_coef, scale;               /* attention */
+    int32_t decay_rank;                     /* wkv */
+} axq_layer_config;
+typedef enum { AXQ_COMPUTE_BF16 = 0, AXQ_COMPUTE_F32 = 1 } axq_compute;
+typedef struct {
+    int32_t vocab_size, width, max_positions;
+    int32_t cache_positions;                /* most positions a sequence may reach; 0: max_positions */
+    int32_t num_layers;
+    int32_t loop_start, loop_stop, loop_times; /* layers loop_start .. loop_stop - 1 run loop_times times in a row, each pass
+                                                  with its own cache or state; loop_times <= 1: no loop */
+    int32_t compute;                        /* axq_compute: bf16 products and an f16 KV cache, or true 32-bit throughout */
+    float norm_eps;
+    float logit_softcap;                    /* logits <- cap tanh(logits / cap); 0: none */
+    const axq_layer_config *layers;         /* num_layers */
+} axq_stack_config;
+AXQ_API int axq_model_create_stack(axq_ctx *ctx, const axq_stack_config *cfg, axq_model **out);
+/* A tensor by name, from f32 values (host): layer -1 = "pos" [max_positions, width], "final.norm", "final.norm.b" [width],
+ * "final.norm.alpha" [1], "head" [vocab, width]; a layer's "norm1", "norm1.b", "norm1.alpha", "norm2" likewise, its mixer's
+ * "mix.q" ..., its feed-forward's "mlp.up", "mlp.down", "mlp.act" [4].  Linears ([out, in]) are kept as AXQ_BF16.  rows x cols
+ * must be the tensor's shape (rows = 1 for vectors).  The embedding goes through axq_model_set_embedding_f32 / _f16. */
+AXQ_API int axq_model_set_tensor(axq_model *m, int layer, const char *name, const float *data, int64_t rows, int64_t cols);
 
 /* ---- next-token selection: TextGenerator::get_next_token (llm/src/generation.rs:258-269) =
  *      apply_repetition_penalty (:145-158, once per occurrence), apply_temperature (:136-142),
