@@ -78,7 +78,9 @@ struct axq_linstate {
     int ldq, ldk, ldv, ldw;
     const float *decay, *u;
     float *state, *o; // o [m][heads * dv]
+    float *seg_state, *seg_decay; // scratch of a prompt cut into segments: AXQ_LINSTATE_SEGS x [heads][dk][dv], x [heads][dk]
 };
+#define AXQ_LINSTATE_SEGS 16
 int axq_linstate_rows(axq_ctx *ctx, const axq_linstate &a, int m, bool first);
 // one token; with `norm_w` each head's o is divided by its root mean square and multiplied by norm_w and gate
 struct axq_linstate_step {

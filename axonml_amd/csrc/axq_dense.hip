@@ -1,8 +1,6 @@
 // Products with bfloat16 weights: the GEMV of a decode step (input transforms, activations and residual adds ride in
 // it) and the GEMM of many rows (bf16 rows on the matrix pipe, or f32 rows in true 32-bit), both over several weights
 // per launch; and the row operations of a prompt around them.
-#include <hip/hip_bf16.h>
-
 #include "axq_dense.h"
 
 namespace {
@@ -16,10 +14,13 @@ typedef __attribute__((address_space(3))) void lds_void;
 __device__ inline float tanh_norm(float x, float alpha, float w, float b) { return tanhf(alpha * x) * w + b; }
 
 // ---------------------------------------------------------------------------------------------------------------------
-// GEMV.  A workgroup stages f(x) in LDS once per distinct input and walks a contiguous range of row blocks (4 R rows,
-// R per wave); a lane's step is 16 bytes (8 weights) of each of its R rows.  x lies in LDS as two planes, elements
-// 8c .. 8c + 3 and 8c + 4 .. 8c + 7 of every chunk c, so that both 16-byte reads of a wave are free of bank conflicts.
+// GEMV.  A workgroup (eight waves) stages f(x) in LDS once per distinct input and walks a contiguous range of row blocks
+// (8 R rows, R per wave); a lane's step is 16 bytes (8 weights) of each of its R rows, U steps make an item.  The next
+// item's weights are requested before the current one is worked on, the first one's before x is staged.  x lies in LDS
+// as two planes, elements 8c .. 8c + 3 and 8c + 4 .. 8c + 7 of every chunk c, so that both 16-byte reads of a wave are
+// free of bank conflicts.
 // ---------------------------------------------------------------------------------------------------------------------
+constexpr int GT = 512, GW = GT / 64; // threads and waves of a workgroup
 struct GemvArgs {
     axq_parts parts;
     axq_in in;
@@ -33,17 +34,17 @@ __device__ void stage_x(const GemvArgs &a, const float *mu, float *xs, float *sc
     auto slot = [half](int e) { return ((e >> 3) << 2) + (e & 3) + ((e & 4) ? half : 0); };
     if (MODE == AXQ_IN_RMS_GATE) {
         float ss = 0.f;
-        for (int e = tid; e < k; e += 256) {
+        for (int e = tid; e < k; e += GT) {
             const float v = in.x[e];
             xs[slot(e)] = v;
             ss = fmaf(v, v, ss);
         }
         ss = axq_block_sum(ss, scratch);
         const float inv = 1.0f / sqrtf(ss / (float)k + in.eps);
-        for (int e = tid; e < xl; e += 256) xs[slot(e)] = e < k ? xs[slot(e)] * inv * in.nw[e] * in.gate[e] : 0.f;
+        for (int e = tid; e < xl; e += GT) xs[slot(e)] = e < k ? xs[slot(e)] * inv * in.nw[e] * in.gate[e] : 0.f;
     } else if (MODE == AXQ_IN_POLY_NORM) {
         float s1 = 0.f, s2 = 0.f, s3 = 0.f;
-        for (int e = tid; e < k; e += 256) {
+        for (int e = tid; e < k; e += GT) {
             const float z = in.x[e], z2 = z * z, z3 = z2 * z;
             xs[slot(e)] = z;
             s1 += z2; s2 = fmaf(z2, z2, s2); s3 = fmaf(z3, z3, s3);
@@ -53,14 +54,14 @@ __device__ void stage_x(const GemvArgs &a, const float *mu, float *xs, float *sc
         s3 = axq_block_sum(s3, scratch);
         const float c1 = in.coef[0] / sqrtf(s1 / (float)k + in.eps), c2 = in.coef[1] / sqrtf(s2 / (float)k + in.eps);
         const float c3 = in.coef[2] / sqrtf(s3 / (float)k + in.eps), c0 = in.coef[3];
-        for (int e = tid; e < xl; e += 256) {
+        for (int e = tid; e < xl; e += GT) {
             const float z = e < k ? xs[slot(e)] : 0.f;
             xs[slot(e)] = e < k ? fmaf(fmaf(fmaf(c3, z, c2), z, c1), z, c0) : 0.f;
         }
     } else {
         const float alpha = MODE == AXQ_IN_PLAIN ? 0.f : in.alpha[0];
         const bool first = MODE == AXQ_IN_TANH_NORM_MIX && in.pos[0] == 0;
-        for (int e = tid; e < xl; e += 256) {
+        for (int e = tid; e < xl; e += GT) {
             float v = 0.f;
             if (e < k) {
                 v = in.x[e];
@@ -77,69 +78,98 @@ __device__ void stage_x(const GemvArgs &a, const float *mu, float *xs, float *sc
 }
 
 template <int MODE, int R>
-__global__ void __launch_bounds__(256) dense_gemv_kernel(GemvArgs a) {
+__global__ void __launch_bounds__(GT, 4) dense_gemv_kernel(GemvArgs a) {
     extern __shared__ __attribute__((aligned(16))) float xs[];
     __shared__ float scratch[16];
     constexpr int U = 8 / R;
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
     const int nb = a.parts.n_blocks, b0 = (int)((long long)nb * blockIdx.x / gridDim.x), b1 = (int)((long long)nb * (blockIdx.x + 1) / gridDim.x);
     const int half = a.steps * 256, k8 = (a.in.k + 7) >> 3;
-    int staged = -1;
-    for (int b = b0; b < b1; b++) {
+    auto part_of_block = [&](int b) {
         int pi = 0;
         while (pi + 1 < a.parts.n_parts && b >= a.parts.p[pi + 1].blk0) pi++;
+        return pi;
+    };
+    // chunks past a row's end: a valid chunk against zeros; rows past the end: the last row, dropped
+    auto request = [&](int b, int s0, u32x4 (&q)[U][R]) {
+        const axq_part &p = a.parts.p[part_of_block(b)];
+        const int row0 = ((b - p.blk0) * GW + wave) * R;
+#pragma unroll
+        for (int r = 0; r < R; r++) {
+            const int row = row0 + r < p.n ? row0 + r : p.n - 1;
+            const uint16_t *w = p.w + (size_t)row * p.ldw;
+#pragma unroll
+            for (int u = 0; u < U; u++) {
+                int c = (s0 + u) * 64 + lane;
+                c = c < k8 ? c : k8 - 1;
+                q[u][r] = __builtin_nontemporal_load(reinterpret_cast<const u32x4 *>(w + (size_t)c * 8));
+            }
+        }
+    };
+    u32x4 qa[U][R], qb[U][R];
+    float acc[R];
+#pragma unroll
+    for (int r = 0; r < R; r++) acc[r] = 0.f;
+    int staged = -1;
+    // one item: the products of block b from step s0 on, and at the row's end the results
+    auto work = [&](int b, int s0, const u32x4 (&q)[U][R]) {
+        const int pi = part_of_block(b);
         const axq_part &p = a.parts.p[pi];
-        if (staged < 0 || (MODE == AXQ_IN_TANH_NORM_MIX && staged != pi)) {
+        if (staged < 0 || (MODE == AXQ_IN_TANH_NORM_MIX && staged != pi)) { // the same for all waves
             if (staged >= 0) __syncthreads();
             stage_x<MODE>(a, p.mu, xs, scratch);
             staged = pi;
         }
-        const int row0 = (b - p.blk0) * 4 * R + wave * R;
-        const uint16_t *w[R];
-        float acc[R];
 #pragma unroll
-        for (int r = 0; r < R; r++) {
-            const int row = row0 + r < p.n ? row0 + r : p.n - 1;
-            w[r] = p.w + (size_t)row * p.ldw;
-            acc[r] = 0.f;
-        }
-        for (int s0 = 0; s0 < a.steps; s0 += U) {
-            u32x4 q[U][R];
+        for (int u = 0; u < U; u++) {
+            if (s0 + u < a.steps) {
+                const int c = (s0 + u) * 64 + lane;
+                const float4 xa = *reinterpret_cast<const float4 *>(xs + c * 4), xb = *reinterpret_cast<const float4 *>(xs + half + c * 4);
 #pragma unroll
-            for (int u = 0; u < U; u++) {
-                int c = (s0 + u) * 64 + lane; // past the row's end: a valid chunk against zeros
-                c = c < k8 ? c : k8 - 1;
-#pragma unroll
-                for (int r = 0; r < R; r++) q[u][r] = __builtin_nontemporal_load(reinterpret_cast<const u32x4 *>(w[r] + (size_t)c * 8));
-            }
-#pragma unroll
-            for (int u = 0; u < U; u++) {
-                if (s0 + u < a.steps) {
-                    const int c = (s0 + u) * 64 + lane;
-                    const float4 xa = *reinterpret_cast<const float4 *>(xs + c * 4), xb = *reinterpret_cast<const float4 *>(xs + half + c * 4);
-#pragma unroll
-                    for (int r = 0; r < R; r++) {
-                        float t = acc[r];
-                        t = fmaf(axq_bf16_lo(q[u][r][0]), xa.x, t); t = fmaf(axq_bf16_hi(q[u][r][0]), xa.y, t);
-                        t = fmaf(axq_bf16_lo(q[u][r][1]), xa.z, t); t = fmaf(axq_bf16_hi(q[u][r][1]), xa.w, t);
-                        t = fmaf(axq_bf16_lo(q[u][r][2]), xb.x, t); t = fmaf(axq_bf16_hi(q[u][r][2]), xb.y, t);
-                        t = fmaf(axq_bf16_lo(q[u][r][3]), xb.z, t); t = fmaf(axq_bf16_hi(q[u][r][3]), xb.w, t);
-                        acc[r] = t;
-                    }
+                for (int r = 0; r < R; r++) {
+                    float t = acc[r];
+                    t = fmaf(axq_bf16_lo(q[u][r][0]), xa.x, t); t = fmaf(axq_bf16_hi(q[u][r][0]), xa.y, t);
+                    t = fmaf(axq_bf16_lo(q[u][r][1]), xa.z, t); t = fmaf(axq_bf16_hi(q[u][r][1]), xa.w, t);
+                    t = fmaf(axq_bf16_lo(q[u][r][2]), xb.x, t); t = fmaf(axq_bf16_hi(q[u][r][2]), xb.y, t);
+                    t = fmaf(axq_bf16_lo(q[u][r][3]), xb.z, t); t = fmaf(axq_bf16_hi(q[u][r][3]), xb.w, t);
+                    acc[r] = t;
                 }
             }
         }
+        if (s0 + U >= a.steps) {
 #pragma unroll
-        for (int r = 0; r < R; r++) acc[r] = axq_wave_sum(acc[r]);
-        float v = acc[0];
+            for (int r = 0; r < R; r++) acc[r] = axq_wave_sum(acc[r]);
+            float v = acc[0];
 #pragma unroll
-        for (int r = 1; r < R; r++) v = lane == r ? acc[r] : v;
-        const int row = row0 + lane;
-        if (lane < R && row < p.n) {
-            if (p.bias) v += p.bias[row];
-            v = axq_act(p.act, v, a.parts.cap);
-            p.y[row] = p.add ? p.y[row] + v : v;
+            for (int r = 1; r < R; r++) v = lane == r ? acc[r] : v;
+            const int row = ((b - p.blk0) * GW + wave) * R + lane;
+            if (lane < R && row < p.n) {
+                if (p.bias) v += p.bias[row];
+                v = axq_act(p.act, v, a.parts.cap);
+                p.y[row] = p.add ? p.y[row] + v : v;
+            }
+#pragma unroll
+            for (int r = 0; r < R; r++) acc[r] = 0.f;
         }
+    };
+    auto advance = [&](int &b, int &s0) {
+        s0 += U;
+        if (s0 >= a.steps) { s0 = 0; b++; }
+    };
+    int b = b0, s0 = 0;
+    if (b >= b1) return;
+    request(b, s0, qa);
+    while (true) {
+        int nb1 = b, ns1 = s0;
+        advance(nb1, ns1);
+        if (nb1 < b1) request(nb1, ns1, qb);
+        work(b, s0, qa);
+        if (nb1 >= b1) break;
+        b = nb1; s0 = ns1;
+        advance(b, s0);
+        if (b < b1) request(b, s0, qa);
+        work(nb1, ns1, qb);
+        if (b >= b1) break;
     }
 }
 
@@ -148,7 +178,7 @@ int launch_gemv(axq_ctx *ctx, GemvArgs &a) {
     int nb = 0;
     for (int i = 0; i < a.parts.n_parts; i++) {
         a.parts.p[i].blk0 = nb;
-        nb += (a.parts.p[i].n + 4 * R - 1) / (4 * R);
+        nb += (a.parts.p[i].n + GW * R - 1) / (GW * R);
     }
     a.parts.n_blocks = nb;
     const int most = 2 * ctx->prop.multiProcessorCount;
@@ -158,7 +188,7 @@ int launch_gemv(axq_ctx *ctx, GemvArgs &a) {
     if (lds > 48 * 1024 &&
         (rc = axq_allow_lds(ctx, reinterpret_cast<const void *>(&dense_gemv_kernel<MODE, R>), lds_allowed, (size_t)AXQ_DENSE_MAX_K * 4)))
         return rc;
-    dense_gemv_kernel<MODE, R><<<nb < most ? nb : most, 256, lds, ctx->stream>>>(a);
+    dense_gemv_kernel<MODE, R><<<nb < most ? nb : most, GT, lds, ctx->stream>>>(a);
     AXQ_LAUNCH_CHECK(ctx, "dense_gemv_kernel");
     return AXQ_OK;
 }
@@ -167,8 +197,7 @@ template <int MODE>
 int launch_gemv_mode(axq_ctx *ctx, GemvArgs &a) {
     long long rows = 0;
     for (int i = 0; i < a.parts.n_parts; i++) rows += a.parts.p[i].n;
-    if (rows >= 8192) return launch_gemv<MODE, 4>(ctx, a);
-    if (rows >= 4096) return launch_gemv<MODE, 2>(ctx, a);
+    if (rows >= 8192) return launch_gemv<MODE, 2>(ctx, a);
     return launch_gemv<MODE, 1>(ctx, a);
 }
 

@@ -4,7 +4,9 @@
 //
 // The columns of S do not depend on each other, so a workgroup takes 16 columns of one head; a column lies across 16
 // lanes, every lane keeping dk / 16 of its elements in registers for the whole prompt.  Tokens come through LDS in
-// blocks; the next block is requested while the current one is worked on.
+// blocks; the next block is requested while the current one is worked on.  Where heads x columns do not fill the chip, the
+// prompt is cut into segments: their states from zero, a scan over them (the update is linear in the state), then all
+// segments side by side from the states they start in.
 #include "axq_dense.h"
 
 namespace {
@@ -37,20 +39,29 @@ __device__ inline void load_elems(const float *row, int g, float (&out)[E]) {
     }
 }
 
-template <int E, bool TOKEN_DECAY>
-__global__ void __launch_bounds__(256) linstate_rows_kernel(axq_linstate a, int m, int first) {
-    constexpr int DKP = 16 * E, NV = TOKEN_DECAY ? 3 : 2, TB = E <= 8 ? 16 : (E <= 12 ? 8 : 4);
-    constexpr int LOADS = (NV * TB * DKP + 255) / 256; // per thread and block
+// Tokens of a group are independent but for the state: their vectors are read ahead, their outputs reduced together.
+template <int E, bool TOKEN_DECAY, bool STATE_ONLY, bool VEC>
+__global__ void __launch_bounds__(256) linstate_rows_kernel(axq_linstate a, int m_all, int first, int seg_len) {
+    constexpr int DKP = 16 * E, NV = TOKEN_DECAY ? 3 : 2, G = E <= (TOKEN_DECAY ? 5 : 8) ? 4 : 2, TB = E <= 8 ? 16 : (E <= 12 ? 8 : 4);
+    constexpr int W = VEC ? 4 : 1, LOADS = (NV * TB * DKP / W + 255) / 256; // per thread and block
     __shared__ __attribute__((aligned(16))) float vec[2][NV][TB][DKP];
-    __shared__ float val[2][TB][16], os[TB][16];
+    __shared__ __attribute__((aligned(16))) float val[2][16][TB], os[16][TB + 1]; // by column
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, g = lane & 15, cw = lane >> 4;
     const int head = blockIdx.x, c0 = blockIdx.y * 16, mycol = wave * 4 + cw, col = c0 + mycol;
     const bool live = col < a.dv;
-    const float *q = a.q + (size_t)head * a.dk, *k = a.k + (size_t)head * a.dk, *v = a.v + (size_t)head * a.dv;
-    const float *wt = TOKEN_DECAY ? a.wt + (size_t)head * a.dk : nullptr;
-    float *st = a.state + (size_t)head * a.dk * a.dv;
+    const int seg = blockIdx.z, t_beg = seg * seg_len, m = m_all - t_beg < seg_len ? m_all - t_beg : seg_len;
+    const float *q = a.q + (size_t)t_beg * a.ldq + (size_t)head * a.dk, *k = a.k + (size_t)t_beg * a.ldk + (size_t)head * a.dk;
+    const float *v = a.v + (size_t)t_beg * a.ldv + (size_t)head * a.dv;
+    const float *wt = TOKEN_DECAY ? a.wt + (size_t)t_beg * a.ldw + (size_t)head * a.dk : nullptr;
+    const size_t head_state = (size_t)head * a.dk * a.dv, all_states = (size_t)a.heads * a.dk * a.dv;
+    float *o_out = a.o + (size_t)t_beg * a.heads * a.dv;
+    const bool cut = STATE_ONLY || seg_len < m_all;
+    float *st = (cut ? a.seg_state + seg * all_states : a.state) + head_state;
+    first = STATE_ONLY || (first && !cut); // of several segments each starts in a state of its own
 
-    float S[E], u[E];
+    float S[E], u[E], wp[STATE_ONLY ? E : 1];
+#pragma unroll
+    for (int i = 0; i < (STATE_ONLY ? E : 1); i++) wp[i] = 1.f;
 #pragma unroll
     for (int i = 0; i < E; i++) {
         const int e = elem_of<E>(g, i);
@@ -59,28 +70,80 @@ __global__ void __launch_bounds__(256) linstate_rows_kernel(axq_linstate a, int 
     }
     const float decay = TOKEN_DECAY ? 0.f : a.decay[head];
 
-    float pre[LOADS], prev_v;
+    // tokens beyond the last: k = 0 and a decay of 1 leave the state as it is
+    float pre[LOADS][W], pre_v;
     auto request = [&](int t0) {
 #pragma unroll
         for (int i = 0; i < LOADS; i++) {
-            const int idx = tid + i * 256, e = idx % DKP, r = idx / DKP, t = t0 + r % TB, which = r / TB;
-            float x = 0.f;
-            if (which < NV && t < m && e < a.dk) {
-                if (which == 0) x = q[(size_t)t * a.ldq + e];
-                else if (which == 1) x = k[(size_t)t * a.ldk + e];
-                else x = wt[(size_t)t * a.ldw + e];
+            const int idx = (tid + i * 256) * W, e = idx % DKP, r = idx / DKP, t = t0 + r % TB, which = r / TB;
+            const bool there = which < NV && t < m && e < a.dk;
+            const float *src = which == 0 ? q + (size_t)t * a.ldq + e : k + (size_t)t * a.ldk + e;
+            if constexpr (TOKEN_DECAY) src = which == 2 ? wt + (size_t)t * a.ldw + e : src;
+            const float none = TOKEN_DECAY && which == 2 ? 1.f : 0.f;
+            if (VEC) {
+                const float4 x = there ? *reinterpret_cast<const float4 *>(src) : make_float4(none, none, none, none);
+                pre[i][0] = x.x; pre[i][1 % W] = x.y; pre[i][2 % W] = x.z; pre[i][3 % W] = x.w;
+            } else {
+                pre[i][0] = there ? *src : none;
             }
-            pre[i] = x;
         }
         const int t = t0 + (tid >> 4), c = c0 + (tid & 15);
-        prev_v = (tid < TB * 16 && t < m && c < a.dv) ? v[(size_t)t * a.ldv + c] : 0.f;
+        pre_v = (tid < TB * 16 && t < m && c < a.dv) ? v[(size_t)t * a.ldv + c] : 0.f;
     };
     auto deposit = [&](int stage) {
         float *dst = &vec[stage][0][0][0];
 #pragma unroll
-        for (int i = 0; i < LOADS; i++)
-            if (tid + i * 256 < NV * TB * DKP) dst[tid + i * 256] = pre[i];
-        if (tid < TB * 16) val[stage][tid >> 4][tid & 15] = prev_v;
+        for (int i = 0; i < LOADS; i++) {
+            const int idx = (tid + i * 256) * W;
+            if (idx < NV * TB * DKP) {
+                if (VEC) *reinterpret_cast<float4 *>(dst + idx) = make_float4(pre[i][0], pre[i][1 % W], pre[i][2 % W], pre[i][3 % W]);
+                else dst[idx] = pre[i][0];
+            }
+        }
+        if (tid < TB * 16) val[stage][tid & 15][tid >> 4] = pre_v;
+    };
+    struct Group { float q[G][STATE_ONLY ? 1 : E], k[G][E], w[G][TOKEN_DECAY ? E : 1], v[G]; };
+    auto read = [&](int stage, int t, Group &x) {
+#pragma unroll
+        for (int i = 0; i < G; i++) {
+            if constexpr (!STATE_ONLY) load_elems<E>(vec[stage][0][t + i], g, x.q[i]);
+            load_elems<E>(vec[stage][1][t + i], g, x.k[i]);
+            if constexpr (TOKEN_DECAY) load_elems<E>(vec[stage][NV - 1][t + i], g, x.w[i]);
+            x.v[i] = val[stage][mycol][t + i];
+        }
+    };
+    auto work = [&](int t, int nt, const Group &x) {
+        float o[G];
+#pragma unroll
+        for (int j = 0; j < G; j++) {
+            float s = 0.f;
+            const bool token = TOKEN_DECAY || t + j < nt; // a constant decay must not touch the state beyond the last token
+#pragma unroll
+            for (int i = 0; i < E; i++) {
+                const float kv = x.k[j][i] * x.v[j];
+                if constexpr (STATE_ONLY) {
+                    float w = decay; // segments of a state-only pass are whole blocks
+                    if constexpr (TOKEN_DECAY) w = x.w[j][i];
+                    S[i] = fmaf(w, S[i], kv);
+                    wp[i] *= w;
+                } else if constexpr (TOKEN_DECAY) {
+                    s = fmaf(x.q[j][i], fmaf(u[i], kv, S[i]), s);
+                    S[i] = fmaf(x.w[j][i], S[i], kv);
+                } else {
+                    S[i] = fmaf(token ? decay : 1.f, S[i], kv);
+                    s = fmaf(x.q[j][i], S[i], s);
+                }
+            }
+            o[j] = s;
+        }
+        if constexpr (!STATE_ONLY) {
+#pragma unroll
+            for (int j = 0; j < G; j++) o[j] = row_sum16(o[j]);
+            if (g == 0) {
+#pragma unroll
+                for (int j = 0; j < G; j++) os[mycol][t + j] = o[j];
+            }
+        }
     };
     request(0);
     deposit(0);
@@ -88,51 +151,74 @@ __global__ void __launch_bounds__(256) linstate_rows_kernel(axq_linstate a, int 
     for (int t0 = 0, stage = 0; t0 < m; t0 += TB, stage ^= 1) {
         if (t0 + TB < m) request(t0 + TB);
         const int nt = m - t0 < TB ? m - t0 : TB;
-        for (int t = 0; t < nt; t++) {
-            float qe[E], ke[E];
-            load_elems<E>(vec[stage][0][t], g, qe);
-            load_elems<E>(vec[stage][1][t], g, ke);
-            const float vv = val[stage][t][mycol];
-            float o = 0.f;
-            if (TOKEN_DECAY) {
-                float we[E];
-                load_elems<E>(vec[stage][NV - 1][t], g, we);
+        Group ga, gb;
+        read(stage, 0, ga);
 #pragma unroll
-                for (int i = 0; i < E; i++) {
-                    const float kv = ke[i] * vv;
-                    o = fmaf(qe[i], fmaf(u[i], kv, S[i]), o);
-                    S[i] = fmaf(we[i], S[i], kv);
-                }
-            } else {
-#pragma unroll
-                for (int i = 0; i < E; i++) {
-                    S[i] = fmaf(decay, S[i], ke[i] * vv);
-                    o = fmaf(qe[i], S[i], o);
-                }
-            }
-            o = row_sum16(o);
-            if (g == 0) os[t][mycol] = o;
+        for (int t = 0; t < TB; t += 2 * G) {
+            read(stage, t + G, gb);
+            work(t, nt, ga);
+            if (t + 2 * G < TB) read(stage, t + 2 * G, ga);
+            work(t + G, nt, gb);
         }
         if (t0 + TB < m) deposit(stage ^ 1);
         __syncthreads(); // the outputs are complete, the next block is in place
-        if (tid < nt * 16 && c0 + (tid & 15) < a.dv)
-            a.o[(size_t)(t0 + (tid >> 4)) * a.heads * a.dv + (size_t)head * a.dv + c0 + (tid & 15)] = os[tid >> 4][tid & 15];
+        if (!STATE_ONLY && tid < nt * 16 && c0 + (tid & 15) < a.dv)
+            o_out[(size_t)(t0 + (tid >> 4)) * a.heads * a.dv + (size_t)head * a.dv + c0 + (tid & 15)] = os[tid & 15][tid >> 4];
         __syncthreads();
+    }
+    if (!STATE_ONLY && cut) {
+        if (t_beg + m < m_all) return;
+        st = a.state + head_state; // the last segment leaves the state behind
     }
 #pragma unroll
     for (int i = 0; i < E; i++) {
         const int e = elem_of<E>(g, i);
         if (live && e < a.dk) st[(size_t)e * a.dv + col] = S[i];
+        if constexpr (STATE_ONLY)
+            if (col == 0 && e < a.dk) a.seg_decay[((size_t)seg * a.heads + head) * a.dk + e] = wp[i];
     }
+}
+
+// seg_state[s] <- the state segment s starts in, given the segments' own contributions
+__global__ void __launch_bounds__(256) linstate_scan_kernel(axq_linstate a, int segs, int first) {
+    const size_t n = (size_t)a.heads * a.dk * a.dv, i = (size_t)blockIdx.x * 256 + threadIdx.x;
+    if (i >= n) return;
+    const size_t hk = i / a.dv;
+    float run = first ? 0.f : a.state[i];
+    for (int s = 0; s < segs; s++) {
+        const float own = s + 1 < segs ? a.seg_state[s * n + i] : 0.f, w = s + 1 < segs ? a.seg_decay[(size_t)s * a.heads * a.dk + hk] : 0.f;
+        a.seg_state[s * n + i] = run;
+        run = fmaf(w, run, own);
+    }
+}
+
+template <int E, bool TOKEN_DECAY, bool VEC>
+int launch_rows_t(axq_ctx *ctx, const axq_linstate &a, int m, bool first, int segs) {
+    const int cols = (a.dv + 15) / 16, len = segs > 1 ? ((m + segs - 1) / segs + 15) / 16 * 16 : m;
+    segs = (m + len - 1) / len;
+    if (segs > 1) {
+        linstate_rows_kernel<E, TOKEN_DECAY, true, VEC><<<dim3(a.heads, cols, segs - 1), 256, 0, ctx->stream>>>(a, m, 1, len);
+        linstate_scan_kernel<<<(unsigned)(((size_t)a.heads * a.dk * a.dv + 255) / 256), 256, 0, ctx->stream>>>(a, segs, first ? 1 : 0);
+    }
+    linstate_rows_kernel<E, TOKEN_DECAY, false, VEC><<<dim3(a.heads, cols, segs), 256, 0, ctx->stream>>>(a, m, first ? 1 : 0, len);
+    AXQ_LAUNCH_CHECK(ctx, "linstate_rows_kernel");
+    return AXQ_OK;
 }
 
 template <int E>
 int launch_rows(axq_ctx *ctx, const axq_linstate &a, int m, bool first) {
-    const dim3 grid(a.heads, (a.dv + 15) / 16);
-    if (a.wt) linstate_rows_kernel<E, true><<<grid, 256, 0, ctx->stream>>>(a, m, first ? 1 : 0);
-    else linstate_rows_kernel<E, false><<<grid, 256, 0, ctx->stream>>>(a, m, first ? 1 : 0);
-    AXQ_LAUNCH_CHECK(ctx, "linstate_rows_kernel");
-    return AXQ_OK;
+    const int wgs = a.heads * ((a.dv + 15) / 16);
+    int segs = 1;
+    if (a.seg_state && wgs < ctx->prop.multiProcessorCount) {
+        segs = 2 * ctx->prop.multiProcessorCount / wgs;
+        if (segs > m / 64) segs = m / 64;
+        if (segs > AXQ_LINSTATE_SEGS) segs = AXQ_LINSTATE_SEGS;
+        if (segs < 1) segs = 1;
+    }
+    auto aligned = [](const void *p, int ld) { return (reinterpret_cast<uintptr_t>(p) & 15) == 0 && ld % 4 == 0; };
+    const bool vec = a.dk % 4 == 0 && aligned(a.q, a.ldq) && aligned(a.k, a.ldk) && (!a.wt || aligned(a.wt, a.ldw));
+    if (a.wt) return vec ? launch_rows_t<E, true, true>(ctx, a, m, first, segs) : launch_rows_t<E, true, false>(ctx, a, m, first, segs);
+    return vec ? launch_rows_t<E, false, true>(ctx, a, m, first, segs) : launch_rows_t<E, false, false>(ctx, a, m, first, segs);
 }
 
 // One token.  grid (heads, column blocks of CB): thread = (column, group of key elements); with a head norm one
@@ -142,52 +228,72 @@ struct StepArgs {
     int cb;
 };
 
+constexpr int TOKEN_PRE = 16; // state elements a thread requests before anything else
+
 __global__ void __launch_bounds__(512) linstate_token_kernel(StepArgs sa) {
     const axq_linstate_step &s = sa.s;
     const axq_linstate &a = s.a;
     extern __shared__ float sm[];
     __shared__ float scratch[16];
-    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, nwave = blockDim.x >> 6, head = blockIdx.x;
+    const int tid = threadIdx.x, head = blockIdx.x;
     const int c0 = blockIdx.y * sa.cb, nc = a.dv - c0 < sa.cb ? a.dv - c0 : sa.cb;
     float *qs = sm, *ks = qs + a.dk, *ws = ks + a.dk, *us = ws + a.dk, *part = us + a.dk; // part [groups][cb]
     const bool first = s.pos[0] == 0;
+    const int col = tid % sa.cb, grp = tid / sa.cb, ngrp = blockDim.x / sa.cb;
+    const bool live = grp < ngrp && col < nc;
+    float *st = a.state + (size_t)head * a.dk * a.dv + c0 + (live ? col : 0);
+    float old[TOKEN_PRE];
+#pragma unroll
+    for (int i = 0; i < TOKEN_PRE; i++) {
+        const int e = grp + i * ngrp;
+        old[i] = (!first && live && e < a.dk) ? st[(size_t)e * a.dv] : 0.f;
+    }
+    const float vv = live ? a.v[(size_t)head * a.dv + c0 + col] : 0.f;
     for (int e = tid; e < a.dk; e += blockDim.x) {
         qs[e] = a.q[(size_t)head * a.dk + e];
         ks[e] = a.k[(size_t)head * a.dk + e];
         us[e] = a.u ? a.u[(size_t)head * a.dk + e] : 0.f;
         if (!s.t1) ws[e] = a.decay[head];
     }
-    if (s.t1) { // w = exp(-exp(W2 t1 + w0)), a wave per key channel
-        for (int e = wave; e < a.dk; e += nwave) {
-            const uint16_t *row = s.w2 + (size_t)(head * a.dk + e) * s.ldw2;
+    if (s.t1) { // w = exp(-exp(W2 t1 + w0)), eight lanes per key channel, 16 bytes of its row at a time
+        const int sub = tid & 7;
+        for (int e0 = 0; e0 < a.dk; e0 += blockDim.x >> 3) {
+            const int e = e0 + (tid >> 3);
             float z = 0.f;
-            for (int r = lane; r < s.rank; r += 64) z = fmaf(axq_bf16_lo(row[r]), s.t1[r], z);
-            z = axq_wave_sum(z);
-            if (lane == 0) ws[e] = expf(-expf(z + s.w0[(size_t)head * a.dk + e]));
+            if (e < a.dk) {
+                const uint16_t *row = s.w2 + (size_t)(head * a.dk + e) * s.ldw2;
+                for (int r = sub * 8; r < s.rank; r += 64) {
+                    const uint4 w = *reinterpret_cast<const uint4 *>(row + r);
+                    const uint32_t ww[4] = {w.x, w.y, w.z, w.w};
+#pragma unroll
+                    for (int i = 0; i < 8; i++)
+                        if (r + i < s.rank) z = fmaf(i & 1 ? axq_bf16_hi(ww[i >> 1]) : axq_bf16_lo(ww[i >> 1]), s.t1[r + i], z);
+                }
+            }
+            z += __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, z), 0xB1, 0xf, 0xf, true));
+            z += __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, z), 0x4E, 0xf, 0xf, true));
+            z += __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, z), 0x141, 0xf, 0xf, true));
+            if (e < a.dk && sub == 0) ws[e] = expf(-expf(z + s.w0[(size_t)head * a.dk + e]));
         }
     }
     __syncthreads();
-    const int col = tid % sa.cb, grp = tid / sa.cb, ngrp = blockDim.x / sa.cb;
     float o = 0.f;
-    if (grp < ngrp && col < nc) {
-        const float vv = a.v[(size_t)head * a.dv + c0 + col];
-        float *st = a.state + (size_t)head * a.dk * a.dv + c0 + col;
-        for (int e0 = grp; e0 < a.dk; e0 += 4 * ngrp) {
-            float old[4];
+    auto update = [&](int e, float before) {
+        const float kv = ks[e] * vv, now = fmaf(ws[e], before, kv);
+        o = fmaf(qs[e], a.u ? fmaf(us[e], kv, before) : now, o);
+        st[(size_t)e * a.dv] = now;
+    };
+    if (live) {
 #pragma unroll
-            for (int i = 0; i < 4; i++) {
-                const int e = e0 + i * ngrp;
-                old[i] = (!first && e < a.dk) ? st[(size_t)e * a.dv] : 0.f;
-            }
+        for (int i = 0; i < TOKEN_PRE; i++)
+            if (grp + i * ngrp < a.dk) update(grp + i * ngrp, old[i]);
+        for (int e0 = grp + TOKEN_PRE * ngrp; e0 < a.dk; e0 += 8 * ngrp) {
+            float more[8];
 #pragma unroll
-            for (int i = 0; i < 4; i++) {
-                const int e = e0 + i * ngrp;
-                if (e < a.dk) {
-                    const float kv = ks[e] * vv, nw = fmaf(ws[e], old[i], kv);
-                    o = fmaf(qs[e], a.u ? fmaf(us[e], kv, old[i]) : nw, o);
-                    st[(size_t)e * a.dv] = nw;
-                }
-            }
+            for (int i = 0; i < 8; i++) more[i] = (!first && e0 + i * ngrp < a.dk) ? st[(size_t)(e0 + i * ngrp) * a.dv] : 0.f;
+#pragma unroll
+            for (int i = 0; i < 8; i++)
+                if (e0 + i * ngrp < a.dk) update(e0 + i * ngrp, more[i]);
         }
     }
     if (grp < ngrp) part[grp * sa.cb + col] = o;

@@ -57,6 +57,7 @@ struct axq_stack {
     // activations of `cap` rows
     int cap = 0;
     float *r_h = nullptr, *r_proj = nullptr, *r_o = nullptr, *r_z = nullptr, *r_logits = nullptr;
+    float *r_seg = nullptr, *r_segw = nullptr; // segments of a recurrence
     void *r_x = nullptr, *r_qs = nullptr;
     int logits_cap = 0;
     float *trace = nullptr;
@@ -216,12 +217,12 @@ int reserve_rows(axq_model *m, int rows) {
     int cap = 64;
     while (cap < rows) cap *= 2;
     AXQ_HIP(ctx, hipStreamSynchronize(ctx->stream), AXQ_ERR_DRIVER);
-    for (void **p : {(void **)&s.r_h, (void **)&s.r_proj, (void **)&s.r_o, (void **)&s.r_z, &s.r_x, &s.r_qs}) {
+    for (void **p : {(void **)&s.r_h, (void **)&s.r_proj, (void **)&s.r_o, (void **)&s.r_z, (void **)&s.r_seg, (void **)&s.r_segw, &s.r_x, &s.r_qs}) {
         if (*p) (void)hipFree(*p);
         *p = nullptr;
     }
     s.cap = 0;
-    size_t proj = 0, o = 0, z = 0, x = pad64(s.c.width), qs = 0;
+    size_t proj = 0, o = 0, z = 0, x = pad64(s.c.width), qs = 0, seg = 0, segw = 0;
     for (Layer &l : s.layers) {
         size_t n = 0;
         for (int w : proj_widths(l.c)) n += w;
@@ -238,6 +239,10 @@ int reserve_rows(axq_model *m, int rows) {
             a.heads = l.c.heads; a.dim = l.c.dim; a.f32 = s.f32;
             const size_t b = axq_sig_attn_q_bytes(a, 1);
             qs = b > qs ? b : qs;
+        } else {
+            const size_t w = (size_t)l.c.heads * l.c.dim, n = w * (l.c.mixer == AXQ_MIX_WKV ? l.c.dim : l.c.vdim);
+            seg = n > seg ? n : seg;
+            segw = w > segw ? w : segw;
         }
     }
     hipError_t e = dev_alloc(&s.r_h, (size_t)cap * s.c.width * 4);
@@ -246,6 +251,8 @@ int reserve_rows(axq_model *m, int rows) {
     if (e == hipSuccess) e = dev_alloc(&s.r_z, (size_t)cap * z * 4);
     if (e == hipSuccess) e = dev_alloc(&s.r_x, (size_t)cap * x * (s.f32 ? 4 : 2));
     if (e == hipSuccess) e = dev_alloc(&s.r_qs, (size_t)cap * qs);
+    if (e == hipSuccess) e = dev_alloc(&s.r_seg, seg * AXQ_LINSTATE_SEGS * 4);
+    if (e == hipSuccess) e = dev_alloc(&s.r_segw, segw * AXQ_LINSTATE_SEGS * 4);
     if (e != hipSuccess) return axq_fail(ctx, AXQ_ERR_ALLOCATION_FAILED, "activations for %d rows: %s", cap, hipGetErrorString(e));
     s.cap = cap;
     return AXQ_OK;
@@ -401,6 +408,8 @@ int axq_stack_rows(axq_model *m, const int32_t *toks, int nb, int pos0) {
                 a.ldw = p.widths[5];
                 if ((rc = axq_store_prev(ctx, in, nb, r.prev))) return rc;
             }
+            a.seg_state = s.r_seg;
+            a.seg_decay = s.r_segw;
             if ((rc = axq_linstate_rows(ctx, a, nb, first))) return rc;
             if ((rc = axq_rows_rms_gate(ctx, gate, nb, mix ? c.dim : mo, xo))) return rc;
         }
@@ -484,7 +493,7 @@ void axq_stack_free(axq_model *m) {
         for (void *p : {r.kc, r.vc, (void *)r.state, (void *)r.prev})
             if (p) (void)hipFree(p);
     for (void *p : {(void *)s->proj, (void *)s->o, (void *)s->z, (void *)s->part, s->qs, (void *)s->r_h, (void *)s->r_proj, (void *)s->r_o,
-                    (void *)s->r_z, (void *)s->r_logits, s->r_x, s->r_qs})
+                    (void *)s->r_z, (void *)s->r_logits, (void *)s->r_seg, (void *)s->r_segw, s->r_x, s->r_qs})
         if (p) (void)hipFree(p);
     delete s;
     m->stack = nullptr;

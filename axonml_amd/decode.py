@@ -26,6 +26,9 @@ class DecoderModel:
     """What every decode model offers, whatever its layers are: an axq_model handle, its embedding, its steps, its generation
     and its sampling.  A subclass creates the handle and loads the layers' weights."""
 
+    max_sequences = 64  # what set_batch takes
+    can_rewind = True   # truncate to any length
+
     def __init__(self, ctx, handle, vocab_size, hidden_size):
         self.ctx, self.handle, self.vocab_size, self.hidden_size = ctx, handle, int(vocab_size), int(hidden_size)
 

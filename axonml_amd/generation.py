@@ -150,9 +150,10 @@ def beam_search_generate(model, input_ids, beam_search, max_new_tokens, batched=
     batched (default: when the model can and there are 2..64 beams): every beam lives in a sequence slot of the
     model and one batched step serves all of them; a beam that forks copies its slot (`copy_sequence`).
     Otherwise the model keeps one sequence, and a beam is brought in by rewinding the cache to the prefix it
-    shares with the cached tokens and feeding the rest (`truncate`, `forward_tokens`)."""
+    shares with the cached tokens and feeding the rest (`truncate`, `forward_tokens`); a model whose state cannot be
+    rewound is fed the whole beam anew unless it extends what the state holds."""
     if batched is None:
-        batched = hasattr(model, "forward_batch") and 2 <= beam_search.num_beams <= 64
+        batched = hasattr(model, "forward_batch") and 2 <= beam_search.num_beams <= getattr(model, "max_sequences", 64)
     if batched:
         return _beam_search_batched(model, input_ids, beam_search, max_new_tokens)
     beams = beam_search.init_beams(input_ids)
@@ -169,6 +170,8 @@ def beam_search_generate(model, input_ids, beam_search, max_new_tokens, batched=
             limit = min(len(cached), len(b.tokens) - 1)  # at least the last token is fed: its logits are wanted
             while shared < limit and cached[shared] == b.tokens[shared]:
                 shared += 1
+            if shared < len(cached) and not getattr(model, "can_rewind", True):
+                shared = 0
             model.truncate(shared)
             _, logits = model.forward_tokens(b.tokens[shared:])
             cached = list(b.tokens)

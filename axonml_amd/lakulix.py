@@ -85,3 +85,81 @@ def load(path, dtype="bfloat16", cache_positions=None, ctx=None):
     cfg = loader.load_config()
     loader.load_tensors()
     return build(cfg, loader.get_tensor, loader.shape, dtype, cache_positions, ctx)
+
+
+# ---------------------------------------------------------------------------------------------------------------------
+# Benchmark: random weights at sizes that resemble a real model's layers, beside the LLaMA-shape model of equal size.
+# ---------------------------------------------------------------------------------------------------------------------
+def bench_description(width, n_blocks, positions, vocab=32000):
+    """Blocks of lightning, attention + feed-forward, time mixing, attention + feed-forward, at LLaMA-like proportions."""
+    ff, heads = width * 7 // 2, width // 128
+    att = LayerDescription(ATTENTION, heads, 128, 128, kv_heads=max(1, heads // 4), ff=ff, bias_rows=32, bias_max=128, scale=128 ** -0.5,
+                           q_temp_every=1024, q_temp_coef=0.1)
+    block = [LayerDescription(LIGHTNING, heads, 128, 128), att, LayerDescription(WKV, width // 64, 64, 64, decay_rank=64), att]
+    return StackDescription(vocab_size=vocab, width=width, max_positions=positions, layers=block * n_blocks, norm_eps=1e-5, logit_softcap=30.0)
+
+
+def linear_weights(d):
+    """Elements of all linears a token passes, the head included."""
+    total = d.vocab_size * d.width
+    for l in d.layers:
+        out = l.heads * l.vdim
+        if l.mixer == ATTENTION:
+            n = l.heads * l.dim + l.kv_heads * (l.dim + l.vdim)
+        elif l.mixer == LIGHTNING:
+            n = 2 * l.heads * l.dim + 2 * out
+        else:
+            n = 4 * l.heads * l.dim + l.decay_rank * (1 + l.heads * l.dim // d.width)
+        total += d.width * (n + out + 2 * l.ff)
+    return total
+
+
+def _rates(model, weights, bytes_per_weight, prompt, new_tokens):
+    model.generate(prompt, 4)
+    model.reset()
+    pre, dec = [], []
+    for _ in range(3):
+        _, p, d = model.generate(prompt, new_tokens)
+        model.reset()
+        pre.append(p)
+        dec.append(d)
+    pre_ms, dec_ms = sorted(pre)[1], sorted(dec)[1]
+    tok_s = (new_tokens - 1) / (dec_ms * 1e-3)
+    return {"prefill_tokens_per_s": len(prompt) / (pre_ms * 1e-3), "prefill_tflops": 2.0 * weights * len(prompt) / (pre_ms * 1e-3) / 1e12,
+            "decode_tokens_per_s": tok_s, "decode_ms_per_token": 1e3 / tok_s, "decode_weight_gbps": weights * bytes_per_weight * tok_s / 1e9}
+
+
+def bench(ctx, log=print, widths=(1024, 2048, 4096), blocks=2, prompt_len=2048, new_tokens=128, beside=True):
+    from .decode import QuantizedLlama
+    from .quant import QuantType
+
+    out = []
+    for width in widths:
+        d = bench_description(width, blocks, prompt_len + new_tokens)
+        weights = linear_weights(d)
+        prompt = np.random.default_rng(0).integers(0, d.vocab_size, size=prompt_len, dtype=np.int32)
+        m = StackModel(d, ctx=ctx)
+        m.random_init(0.02, 1)
+        r = {"width": width, "layers": len(d.layers), "linear_weights": weights, "prompt_tokens": prompt_len, "generated_tokens": new_tokens,
+             "lakulix_bf16": _rates(m, weights, 2.0, prompt, new_tokens)}
+        m.close()
+        if beside:
+            heads, ff = width // 128, width * 7 // 2
+            kv = max(1, heads // 4)
+            per_layer = width * (2 * width + 2 * kv * 128 + 3 * ff)
+            n = max(1, round((weights - d.vocab_size * width) / per_layer))
+            cfg = dict(vocab_size=d.vocab_size, hidden_size=width, intermediate_size=ff, num_hidden_layers=n, num_attention_heads=heads,
+                       num_key_value_heads=kv, head_dim=128, max_position_embeddings=prompt_len + new_tokens, rms_norm_eps=1e-5,
+                       rope_theta=10000.0)
+            lw = n * per_layer + d.vocab_size * width
+            for qt, bpw in ((QuantType.BF16, 2.0), (QuantType.Q4_K, 0.5625)):
+                lm = QuantizedLlama(ctx, **cfg)
+                lm.random_init(qt, 0.02, 1)
+                r[f"llama_{str(qt).lower()}"] = dict(_rates(lm, lw, bpw, prompt, new_tokens), layers=n, linear_weights=lw)
+                lm.close()
+        for name, v in r.items():
+            if isinstance(v, dict):
+                log(f"  width {width} {name}: prefill {v['prefill_tokens_per_s']:.0f} tok/s ({v['prefill_tflops']:.0f} TFLOP/s), decode "
+                    f"{v['decode_tokens_per_s']:.0f} tok/s ({v['decode_ms_per_token']:.3f} ms, {v['decode_weight_gbps']:.0f} GB/s of weights)")
+        out.append(r)
+    return out

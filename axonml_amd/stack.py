@@ -51,6 +51,8 @@ class StackDescription:
 
 
 class StackModel(DecoderModel):
+    max_sequences = 1
+
     def __init__(self, description, dtype="bfloat16", cache_positions=None, ctx=None):
         ctx = ctx or default_context()
         self.description, self.dtype = description, dtype
@@ -63,6 +65,7 @@ class StackModel(DecoderModel):
         h = C.c_void_p()
         ctx.check(ctx.lib.axq_model_create_stack(ctx.handle, C.byref(cfg), C.byref(h)))
         super().__init__(ctx, h, d.vocab_size, d.width)
+        self.can_rewind = all(l.mixer == ATTENTION for l in d.layers)
 
     def set_tensor(self, layer, name, data):
         """A weight by its name; layer -1 for those outside the layers."""

@@ -406,6 +406,11 @@ def main():
     ap.add_argument("--gemv-table", action="store_true",
                     help="instead of the benchmark, for kernel-trace profiles: the one-vector and batch-8 GEMVs of every block "
                          "type at 14336x4096 and 4096x14336 as plain stream launches over their rings, one line each")
+    ap.add_argument("--lakulix", action="store_true",
+                    help="instead of the benchmark: prefill and decode throughput of Lakulix models with random weights beside LLaMA-shape "
+                         "models of equal size, as one JSON line")
+    ap.add_argument("--lakulix-widths", default="1024,2048,4096", help="widths of --lakulix")
+    ap.add_argument("--lakulix-only", action="store_true", help="with --lakulix, for kernel profiles: without the LLaMA-shape models")
     ap.add_argument("--grid-barrier", action="store_true",
                     help="instead of the benchmark: time a barrier over all workgroups of one resident launch through device-scope "
                          "atomics (what a kernel that spans dependent steps would pay per step), and print the table")
@@ -435,6 +440,13 @@ def main():
             for pub in (0, 1024, 4096, 16384):
                 ctx.check(lib.axq_bench_grid_barrier(ctx.handle, levels, pub, 256, out))
                 print(f"{'one' if levels == 1 else '16 + 1':8s}  {pub:8d}   {out[0]:6.2f}   {out[1]:6.2f}   {out[2]:6.2f}", flush=True)
+        return
+    if args.lakulix or args.lakulix_only:
+        from axonml_amd import lakulix
+
+        res = lakulix.bench(ctx, log, widths=tuple(int(w) for w in args.lakulix_widths.split(",")), beside=not args.lakulix_only)
+        print(json.dumps({"lakulix": res}), flush=True)
+        ctx.close()
         return
     if args.gemv_table:
         for qt in (T.Q4_K, T.Q5_K, T.Q6_K, T.Q4_0, T.Q4_1, T.Q5_0, T.Q5_1, T.Q8_0):
