@@ -45,13 +45,13 @@ struct axq_in {
     const float *prev = nullptr;    // [k] the previous token's normed input
     const int32_t *pos = nullptr;   // position of this token
     const float *gate = nullptr, *coef = nullptr;
+    const int32_t *rows = nullptr;  // axq_rows_tanh_norm: output row t is input row rows[t] (NULL: t)
 };
 
 #define AXQ_DENSE_MAX_K 36864 // widest input of a decode product (it is staged in LDS)
 
 // One vector against the parts.
 int axq_dense_gemv(axq_ctx *ctx, int mode, const axq_in &in, axq_parts &parts);
-
 // m rows against the parts; k is padded by the caller's rows to ldx = a multiple of 64 with zeros.
 // f32 rows: true 32-bit multiply-adds; bf16 rows: the matrix pipe.
 int axq_dense_gemm(axq_ctx *ctx, axq_parts &parts, int m, int k, int ldx, bool f32);

@@ -391,7 +391,7 @@ struct MixPtrs { const float *mu[AXQ_MAX_PARTS]; };
 __global__ void __launch_bounds__(256) rows_tanh_norm_kernel(axq_in in, int m, int first, int n_mix, MixPtrs mix, axq_rows_out out) {
     const int t = blockIdx.x;
     const float alpha = in.alpha[0];
-    const float *h = in.x + (size_t)t * in.k;
+    const float *h = in.x + (size_t)(in.rows ? in.rows[t] : t) * in.k;
     for (int e = threadIdx.x; e < out.ldx; e += 256) {
         const bool in_row = e < in.k;
         const float nw = in_row ? in.nw[e] : 0.f, nb = in_row ? in.nb[e] : 0.f;

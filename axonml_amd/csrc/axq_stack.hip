@@ -59,6 +59,7 @@ struct axq_stack {
     float *r_h = nullptr, *r_proj = nullptr, *r_o = nullptr, *r_z = nullptr, *r_logits = nullptr;
     float *r_seg = nullptr, *r_segw = nullptr; // segments of a recurrence
     void *r_x = nullptr, *r_qs = nullptr;
+    int32_t *r_want = nullptr;
     int logits_cap = 0;
     float *trace = nullptr;
     int trace_total = 0, trace_row0 = 0;
@@ -457,14 +458,15 @@ int axq_stack_logits_rows(axq_model *m, const int32_t *rows, int n, float *logit
         s.r_logits = nullptr;
         s.logits_cap = 0;
         AXQ_HIP(ctx, dev_alloc(&s.r_logits, (size_t)want * V * 4), AXQ_ERR_ALLOCATION_FAILED);
+        if (!s.r_want) AXQ_HIP(ctx, dev_alloc(&s.r_want, LOGITS_ROWS * 4), AXQ_ERR_ALLOCATION_FAILED);
         s.logits_cap = want;
     }
     for (int j0 = 0; j0 < n; j0 += want) {
         const int nj = n - j0 < want ? n - j0 : want;
-        for (int j = 0; j < nj; j++) {
-            axq_rows_out out = {reinterpret_cast<uint8_t *>(s.r_x) + (size_t)j * ldw * (s.f32 ? 4 : 2), ldw, s.f32};
-            if ((rc = axq_rows_tanh_norm(ctx, norm_in(s, s.top, "final.norm", s.r_h + (size_t)rows[j0 + j] * W), 1, true, 0, nullptr, out))) return rc;
-        }
+        AXQ_HIP(ctx, hipMemcpyAsync(s.r_want, rows + j0, (size_t)nj * 4, hipMemcpyHostToDevice, ctx->stream), AXQ_ERR_COPY_FAILED);
+        axq_in in = norm_in(s, s.top, "final.norm", s.r_h);
+        in.rows = s.r_want;
+        if ((rc = axq_rows_tanh_norm(ctx, in, nj, true, 0, nullptr, {s.r_x, ldw, s.f32}))) return rc;
         axq_parts hd = {};
         hd.n_parts = 1;
         hd.cap = s.c.logit_softcap;
@@ -493,7 +495,7 @@ void axq_stack_free(axq_model *m) {
         for (void *p : {r.kc, r.vc, (void *)r.state, (void *)r.prev})
             if (p) (void)hipFree(p);
     for (void *p : {(void *)s->proj, (void *)s->o, (void *)s->z, (void *)s->part, s->qs, (void *)s->r_h, (void *)s->r_proj, (void *)s->r_o,
-                    (void *)s->r_z, (void *)s->r_logits, (void *)s->r_seg, (void *)s->r_segw, s->r_x, s->r_qs})
+                    (void *)s->r_z, (void *)s->r_logits, (void *)s->r_seg, (void *)s->r_segw, (void *)s->r_want, s->r_x, s->r_qs})
         if (p) (void)hipFree(p);
     delete s;
     m->stack = nullptr;
