@@ -20,6 +20,19 @@ pub struct axq_model_config {
     pub max_position_embeddings: i32, pub rms_norm_eps: f32, pub rope_theta: f32, pub sliding_window: i32,
 }
 
+#[repr(C)]
+pub struct axq_layer_config {
+    pub mixer: i32, pub heads: i32, pub kv_heads: i32, pub dim: i32, pub vdim: i32, pub ff: i32,
+    pub bias_rows: i32, pub bias_max: i32, pub q_temp_every: i32, pub q_temp_coef: f32, pub scale: f32, pub decay_rank: i32,
+}
+
+#[repr(C)]
+pub struct axq_stack_config {
+    pub vocab_size: i32, pub width: i32, pub max_positions: i32, pub cache_positions: i32, pub num_layers: i32,
+    pub loop_start: i32, pub loop_stop: i32, pub loop_times: i32, pub compute: i32, pub norm_eps: f32, pub logit_softcap: f32,
+    pub layers: *const axq_layer_config,
+}
+
 #[link(name = "axq")]
 extern "C" {
     pub fn axq_init(device: c_int, out: *mut *mut axq_ctx) -> c_int;
@@ -67,4 +80,12 @@ extern "C" {
                                     out: *mut i32, prefill_ms: *mut f32, decode_ms: *mut f32) -> c_int;
     pub fn axq_model_generate(m: *mut axq_model, prompt: *const i32, n_prompt: c_int, max_new: c_int,
                               out: *mut i32, prefill_ms: *mut f32, decode_ms: *mut f32) -> c_int;
+    /// Rows of a prompt; logits at the rising places `want`; `layers` (may be null): described layers only.
+    pub fn axq_model_forward_rows(m: *mut axq_model, tokens: *const i32, n: c_int, want: *const i32, n_want: c_int,
+                                  logits: *mut f32, layers: *mut f32) -> c_int;
+    pub fn axq_model_layer_runs(m: *const axq_model) -> c_int;
+
+    pub fn axq_model_create_stack(ctx: *mut axq_ctx, cfg: *const axq_stack_config, out: *mut *mut axq_model) -> c_int;
+    pub fn axq_model_set_tensor(m: *mut axq_model, layer: c_int, name: *const c_char, data: *const f32,
+                                rows: i64, cols: i64) -> c_int;
 }
