@@ -117,6 +117,18 @@ def test_portions_and_reuse(ctx, mixed, dtype):
     m.close()
 
 
+def test_prompt_chunks(ctx, mixed, monkeypatch):
+    """A prompt longer than what goes through the layers at once: wanted places and layer outputs on both sides of every seam."""
+    t, tokens, want, runs = mixed
+    monkeypatch.setenv("AXQ_PROMPT_CHUNK", "50")
+    m = lc.product(MIXED, t, "float32", ctx)
+    places = [0, 48, 49, 50, 51, 99, 100, 149, 150, 151, 298, 300, 329]
+    got, layers = m.forward_rows(tokens, places, layers=True)
+    assert close(got, want[places], "float32", 2)
+    assert np.abs(layers - runs).max() <= 2 * lc.LIMIT["float32"] * np.abs(runs).max()
+    m.close()
+
+
 @pytest.mark.parametrize("dtype", DTYPES)
 def test_long_decoding(ctx, mixed, dtype):
     t, tokens, want, _ = mixed
