@@ -61,13 +61,17 @@ class ModelConfig(C.Structure):
 class LayerConfig(C.Structure):
     _fields_ = [("mixer", C.c_int32), ("heads", C.c_int32), ("kv_heads", C.c_int32), ("dim", C.c_int32), ("vdim", C.c_int32), ("ff", C.c_int32),
                 ("bias_rows", C.c_int32), ("bias_max", C.c_int32), ("q_temp_every", C.c_int32), ("q_temp_coef", C.c_float), ("scale", C.c_float),
-                ("decay_rank", C.c_int32)]
+                ("decay_rank", C.c_int32), ("window", C.c_int32), ("pool", C.c_int32), ("keys_as_values", C.c_int32), ("head_gate", C.c_int32),
+                ("rot_dims", C.c_int32), ("rot_original", C.c_int32), ("rot_base", C.c_double), ("rot_factor", C.c_double),
+                ("rot_fast", C.c_double), ("rot_slow", C.c_double), ("ff_kind", C.c_int32), ("experts", C.c_int32), ("top", C.c_int32),
+                ("groups", C.c_int32), ("groups_keep", C.c_int32), ("shared_ff", C.c_int32)]
 
 
 class StackConfig(C.Structure):
     _fields_ = [("vocab_size", C.c_int32), ("width", C.c_int32), ("max_positions", C.c_int32), ("cache_positions", C.c_int32),
                 ("num_layers", C.c_int32), ("loop_start", C.c_int32), ("loop_stop", C.c_int32), ("loop_times", C.c_int32), ("compute", C.c_int32),
-                ("norm_eps", C.c_float), ("logit_softcap", C.c_float), ("layers", C.POINTER(LayerConfig))]
+                ("norm_eps", C.c_float), ("logit_softcap", C.c_float), ("layers", C.POINTER(LayerConfig)),
+                ("norm", C.c_int32), ("position_table", C.c_int32), ("parallel", C.c_int32), ("depth_average", C.c_int32)]
 
 
 _vp, _sz, _i, _i64 = C.c_void_p, C.c_size_t, C.c_int, C.c_int64

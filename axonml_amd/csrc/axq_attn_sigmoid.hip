@@ -2,30 +2,9 @@
 // queries and keys, a query factor by position and a learned bias by distance:
 //   w_ij = sigmoid(scale (q_i . k_j) + bias[h][min(i - j, nt - 1)]),   o_i = sum_j w_ij v_j.
 // Without a normaliser partial sums over ranges of keys just add up: no running maximum, no rescaling.
-//
-// Cache in f16: keys [kv_head][position][DP] (head size padded with zeros to 64, 128 or 256), values transposed,
-// [kv_head][DVP][position] with positions 4..7 and 8..11 of every 16 exchanged (value_slot), so that both operands of a
-// matrix-pipe tile are 16 contiguous bytes per lane.  In f32: keys and
-// values row-major, products on the vector ALU.
-#include <hip/hip_fp16.h>
-
-#include "axq_dense.h"
+#include "axq_attn_tiles.h"
 
 namespace {
-
-typedef _Float16 half8 __attribute__((ext_vector_type(8)));
-typedef float f32x16 __attribute__((ext_vector_type(16)));
-
-constexpr int CHUNK = 64;      // positions per workgroup of a decode step
-constexpr float PSCALE = 32768.0f; // weights enter the second product as f16 times this: (0, 1] stays normal down to 2^-29
-
-inline int pad_dim(int d) { return d <= 64 ? 64 : (d <= 128 ? 128 : 256); }
-inline int pad_cap(int cap) { return (cap + 63) / 64 * 64; }
-
-__device__ inline _Float16 to_half(float f) { return (_Float16)fminf(fmaxf(f, -65504.f), 65504.f); }
-
-// Where position p of a value row lies: bits 2 and 3 exchanged.
-__device__ inline int value_slot(int p) { return (p & ~12) | ((p & 4) << 1) | ((p & 8) >> 1); }
 
 struct Args {
     axq_sig_attn a;
@@ -85,19 +64,7 @@ __global__ void __launch_bounds__(64) prep_kernel(Args g) {
     }
 }
 
-// Values of a prompt's rows into the transposed f16 cache through LDS: grid (32-position tiles, 32-element tiles, kv
-// heads), so that both sides are runs of 64 bytes or more.
-__global__ void __launch_bounds__(256) append_values_kernel(Args g) {
-    __shared__ float tile[32][33];
-    const axq_sig_attn &a = g.a;
-    const int t0 = blockIdx.x * 32, e0 = blockIdx.y * 32, h = blockIdx.z, x = threadIdx.x & 31, y = threadIdx.x >> 5;
-    for (int i = y; i < 32; i += 8)
-        tile[i][x] = (t0 + i < g.m && e0 + x < a.vdim) ? g.v[(size_t)(t0 + i) * g.ldv + (size_t)h * a.vdim + e0 + x] : 0.f;
-    __syncthreads();
-    _Float16 *o = reinterpret_cast<_Float16 *>(a.vc) + (size_t)h * g.dvp * g.capp;
-    for (int i = y; i < 32; i += 8)
-        if (e0 + i < a.vdim && t0 + x < g.m) o[(size_t)(e0 + i) * g.capp + value_slot(g.pos0 + t0 + x)] = to_half(tile[x][i]);
-}
+__global__ void __launch_bounds__(256) append_values_kernel(Args g) { append_values(g.v, g.ldv, g.a.vdim, g.m, g.pos0, g.a.vc, g.dvp, g.capp); }
 
 // Rows against the f32 cache: grid (heads, rows).  256 keys at a time: scores by thread, then the value sum by element.
 __global__ void __launch_bounds__(256) rows_f32_kernel(Args g, axq_rows_out out) {
@@ -150,11 +117,6 @@ __global__ void __launch_bounds__(256) rows_f32_kernel(Args g, axq_rows_out out)
 // The four waves of a workgroup walk the same keys, 64 at a time, through LDS (two stages, filled straight from memory;
 // the 16-byte pieces of a row are exchanged by row % 8 so that operand reads use all banks).  Workgroups with the longest
 // ranges start first.
-__device__ inline int acc_row(int r, int lane) { return 8 * (r >> 2) + 4 * (lane >> 5) + (r & 3); }
-
-typedef const __attribute__((address_space(1))) void gbl_void;
-typedef __attribute__((address_space(3))) void lds_void;
-
 template <int KS, int DB>
 __global__ void __launch_bounds__(256, KS + DB > 20 ? 1 : 2) rows_mfma_kernel(Args g, axq_rows_out out) {
     constexpr int DP = KS * 16, DVP = DB * 32, KC = DP / 8; // KC: 16-byte pieces of a key row

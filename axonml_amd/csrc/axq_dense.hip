@@ -28,10 +28,47 @@ struct GemvArgs {
 };
 
 template <int MODE>
-__device__ void stage_x(const GemvArgs &a, const float *mu, float *xs, float *scratch) {
+__device__ void stage_x(const GemvArgs &a, const axq_part &p, float *xs, float *scratch) {
     const axq_in &in = a.in;
+    const float *mu = p.mu;
     const int k = in.k, tid = threadIdx.x, xl = a.steps * 512, half = xl >> 1;
     auto slot = [half](int e) { return ((e >> 3) << 2) + (e & 3) + ((e & 4) ? half : 0); };
+    if (MODE == AXQ_IN_SEGMENTS) {
+        for (int s = 0; s < in.n_seg; s++) {
+            const axq_seg &g = in.seg[s];
+            const int span = g.steps * 512;
+            for (int i = 0; i < g.count; i++) {
+                const float *x = g.x + (size_t)i * g.ldx, f = g.scale ? g.scale[i] : 1.0f;
+                const int e0 = (g.step0 + i * g.steps) * 512;
+                for (int e = tid; e < span; e += GT) {
+                    float v = 0.f;
+                    if (e < g.k) {
+                        if (g.glu) {
+                            const float *z = x + (e / AXQ_GLU_GROUP) * 2 * AXQ_GLU_GROUP + e % AXQ_GLU_GROUP;
+                            v = z[0] * z[AXQ_GLU_GROUP];
+                        } else {
+                            v = x[e];
+                        }
+                    }
+                    xs[slot(e0 + e)] = v * f;
+                }
+            }
+        }
+    } else if (MODE == AXQ_IN_LAYER_NORM) {
+        float sum = 0.f, ss = 0.f;
+        for (int e = tid; e < k; e += GT) {
+            const float v = in.x[e];
+            xs[slot(e)] = v;
+            sum += v;
+        }
+        const float mean = axq_block_sum(sum, scratch) / (float)k;
+        for (int e = tid; e < k; e += GT) {
+            const float d = xs[slot(e)] - mean;
+            ss = fmaf(d, d, ss);
+        }
+        const float inv = 1.0f / sqrtf(axq_block_sum(ss, scratch) / (float)k + in.eps);
+        for (int e = tid; e < xl; e += GT) xs[slot(e)] = e < k ? (xs[slot(e)] - mean) * inv * p.nw[e] : 0.f;
+    } else
     if (MODE == AXQ_IN_RMS_GATE) {
         float ss = 0.f;
         for (int e = tid; e < k; e += GT) {
@@ -81,6 +118,9 @@ template <int MODE, int R>
 __global__ void __launch_bounds__(GT, 4) dense_gemv_kernel(GemvArgs a) {
     extern __shared__ __attribute__((aligned(16))) float xs[];
     __shared__ float scratch[16];
+    constexpr bool SEG = MODE == AXQ_IN_SEGMENTS;
+    struct Step { const uint16_t *w; int ldw, c8; }; // of a step: its weight's columns, their row pitch and 16-byte chunks
+    __shared__ Step table[SEG ? AXQ_DENSE_MAX_K / 512 : 1];
     constexpr int U = 8 / R;
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
     const int nb = a.parts.n_blocks, b0 = (int)((long long)nb * blockIdx.x / gridDim.x), b1 = (int)((long long)nb * (blockIdx.x + 1) / gridDim.x);
@@ -90,13 +130,38 @@ __global__ void __launch_bounds__(GT, 4) dense_gemv_kernel(GemvArgs a) {
         while (pi + 1 < a.parts.n_parts && b >= a.parts.p[pi + 1].blk0) pi++;
         return pi;
     };
+    if (SEG) {
+        for (int t = tid; t < a.steps; t += GT) {
+            int si = 0;
+            while (si + 1 < a.in.n_seg && t >= a.in.seg[si + 1].step0) si++;
+            const axq_seg &g = a.in.seg[si];
+            const int i = (t - g.step0) / g.steps, s = (t - g.step0) - i * g.steps;
+            table[t].w = g.w + (size_t)(g.sel ? g.sel[i] : i) * g.stride + (size_t)s * 512;
+            table[t].ldw = g.ldw;
+            table[t].c8 = ((g.k + 7) >> 3) - s * 64;
+        }
+        __syncthreads();
+    }
     // chunks past a row's end: a valid chunk against zeros; rows past the end: the last row, dropped
     auto request = [&](int b, int s0, u32x4 (&q)[U][R]) {
         const axq_part &p = a.parts.p[part_of_block(b)];
         const int row0 = ((b - p.blk0) * GW + wave) * R;
 #pragma unroll
         for (int r = 0; r < R; r++) {
-            const int row = row0 + r < p.n ? row0 + r : p.n - 1;
+            int row = row0 + r < p.n ? row0 + r : p.n - 1;
+            if (SEG) {
+#pragma unroll
+                for (int u = 0; u < U; u++) {
+                    const Step t = table[s0 + u < a.steps ? s0 + u : a.steps - 1];
+                    const int c = lane < t.c8 ? lane : t.c8 - 1;
+                    q[u][r] = __builtin_nontemporal_load(reinterpret_cast<const u32x4 *>(t.w + (size_t)row * t.ldw + (size_t)c * 8));
+                }
+                continue;
+            }
+            if (MODE == AXQ_IN_LAYER_NORM && p.sel) {
+                const int i = row / p.sel_rows;
+                row += (p.sel[i] - i) * p.sel_rows;
+            }
             const uint16_t *w = p.w + (size_t)row * p.ldw;
 #pragma unroll
             for (int u = 0; u < U; u++) {
@@ -115,9 +180,10 @@ __global__ void __launch_bounds__(GT, 4) dense_gemv_kernel(GemvArgs a) {
     auto work = [&](int b, int s0, const u32x4 (&q)[U][R]) {
         const int pi = part_of_block(b);
         const axq_part &p = a.parts.p[pi];
-        if (staged < 0 || (MODE == AXQ_IN_TANH_NORM_MIX && staged != pi)) { // the same for all waves
+        if (staged < 0 || (MODE == AXQ_IN_TANH_NORM_MIX && staged != pi) ||
+            (MODE == AXQ_IN_LAYER_NORM && a.parts.p[staged].nw != p.nw)) { // the same for all waves
             if (staged >= 0) __syncthreads();
-            stage_x<MODE>(a, p.mu, xs, scratch);
+            stage_x<MODE>(a, p, xs, scratch);
             staged = pi;
         }
 #pragma unroll
@@ -145,8 +211,10 @@ __global__ void __launch_bounds__(GT, 4) dense_gemv_kernel(GemvArgs a) {
             const int row = ((b - p.blk0) * GW + wave) * R + lane;
             if (lane < R && row < p.n) {
                 if (p.bias) v += p.bias[row];
-                v = axq_act(p.act, v, a.parts.cap);
-                p.y[row] = p.add ? p.y[row] + v : v;
+                v = p.act == AXQ_ACT_GLU_GELU ? ((row & AXQ_GLU_GROUP) ? v : axq_gelu_tanh(v)) : axq_act(p.act, v, a.parts.cap);
+                if (p.resid) v += p.resid[row];
+                reinterpret_cast<float *>(p.y)[row] = v;
+                if (p.avg.out) p.avg.out[row] = axq_average(p.avg, row, v);
             }
 #pragma unroll
             for (int r = 0; r < R; r++) acc[r] = 0.f;
@@ -210,7 +278,35 @@ int launch_gemv_mode(axq_ctx *ctx, GemvArgs &a) {
 struct GemmArgs {
     axq_parts parts;
     int m, k, ldx, mt, tiles;
+    axq_groups g; // grouped form
 };
+
+// A product's result on its way out (act_done: the activation has been applied)
+__device__ inline void finish(const axq_part &p, float cap, int m, int n, float v, bool act_done = false) {
+    if (p.bias) v += p.bias[n];
+    if (!act_done) v = axq_act(p.act, v, cap);
+    if (p.scale) v *= p.scale[m];
+    const size_t i = (size_t)m * p.ldy + n;
+    if (p.resid) v += p.resid[i];
+    if (p.out16) reinterpret_cast<uint16_t *>(p.y)[i] = axq_to_bf16(v);
+    else reinterpret_cast<float *>(p.y)[i] = v;
+}
+
+// ... and, once a thread's results are written, the mean over the layers at one of them
+__device__ inline void finish_mean(const axq_part &p, int m, int n) {
+    const size_t i = (size_t)m * p.ldy + n;
+    p.avg.out[i] = axq_average(p.avg, i, reinterpret_cast<const float *>(p.y)[i]);
+}
+
+// Which rows and which weight a workgroup of a grouped product has: row tile `t` -> false if there is no such tile.
+__device__ inline bool group_tile(const axq_groups &g, int t, int &m0, int &m1, size_t &woff) {
+    if (t >= g.tiles[0]) return false;
+    const int32_t *e = g.tiles + 4 + 4 * t;
+    woff = (size_t)e[0] * g.stride;
+    m0 = e[1];
+    m1 = e[2];
+    return true;
+}
 
 __device__ inline int acc_row(int r, int lane) { return 8 * (r >> 2) + 4 * (lane >> 5) + (r & 3); }
 
@@ -221,15 +317,17 @@ __device__ inline int xcd_tile(int tiles) {
     return x * per + (x < rest ? x : rest) + (b >> 3);
 }
 
-template <int BM, int BN>
+template <int BM, int BN, bool GROUPED>
 __global__ void __launch_bounds__(256) dense_gemm_kernel(GemmArgs a) {
     constexpr int MT = BM / 64, NT = BN / 64;          // 32 x 32 tiles of a wave (2 x 2 waves)
     constexpr int AL = BM / 32, BL = BN / 32;          // 16-byte loads per thread and step
     __shared__ __attribute__((aligned(16))) uint16_t lds[2][(BM + BN) * 64];
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, wm = wave >> 1, wn = wave & 1;
-    const int tile = xcd_tile(a.tiles), ct = tile / a.mt, m0 = (tile - ct * a.mt) * BM;
-    int pi = 0;
-    while (pi + 1 < a.parts.n_parts && ct >= a.parts.p[pi + 1].blk0) pi++;
+    const int tile = xcd_tile(a.tiles), ct = tile / a.mt;
+    int m0 = (tile - ct * a.mt) * BM, m1 = a.m, pi = 0;
+    size_t woff = 0;
+    if (GROUPED && !group_tile(a.g, tile - ct * a.mt, m0, m1, woff)) return;
+    while (!GROUPED && pi + 1 < a.parts.n_parts && ct >= a.parts.p[pi + 1].blk0) pi++;
     const axq_part &p = a.parts.p[pi];
     const int n0 = (ct - p.blk0) * BN;
     const uint16_t *x = reinterpret_cast<const uint16_t *>(p.x);
@@ -238,14 +336,15 @@ __global__ void __launch_bounds__(256) dense_gemm_kernel(GemmArgs a) {
 #pragma unroll
     for (int i = 0; i < AL; i++) {
         const int idx = (i * 4 + wave) * 64 + lane, r = idx >> 3, c = (idx & 7) ^ (r & 7);
-        const int row = m0 + r < a.m ? m0 + r : a.m - 1;
+        int row = m0 + r < m1 ? m0 + r : m1 - 1;
+        if (GROUPED && a.g.src) row = a.g.src[row];
         ga[i] = x + (size_t)row * a.ldx + c * 8;
     }
 #pragma unroll
     for (int i = 0; i < BL; i++) {
         const int idx = (i * 4 + wave) * 64 + lane, r = idx >> 3, c = (idx & 7) ^ (r & 7);
         const int row = n0 + r < p.n ? n0 + r : p.n - 1;
-        gb[i] = p.w + (size_t)row * p.ldw + c * 8;
+        gb[i] = p.w + woff + (size_t)row * p.ldw + c * 8;
     }
     auto fetch = [&](int stage, int kt) {
         uint16_t *la = lds[stage], *lb = la + BM * 64;
@@ -290,38 +389,57 @@ __global__ void __launch_bounds__(256) dense_gemm_kernel(GemmArgs a) {
                 for (int j = 0; j < NT; j++) acc[i][j] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(fa[i], fb[j], acc[i][j], 0, 0, 0);
         }
     }
-#pragma unroll
-    for (int j = 0; j < NT; j++) {
-        const int n = n0 + wn * (BN / 2) + j * 32 + li;
-        if (n >= p.n) continue;
-        const float bias = p.bias ? p.bias[n] : 0.f;
+    if (NT == 2 && p.act == AXQ_ACT_GLU_GELU) { // a wave's two column tiles are a group of gates and its ups
+        const int n = n0 / 2 + wn * 32 + li;
+        if (n >= p.n / 2) return;
 #pragma unroll
         for (int i = 0; i < MT; i++)
 #pragma unroll
             for (int r = 0; r < 16; r++) {
                 const int m = m0 + wm * (BM / 2) + i * 32 + acc_row(r, lane);
-                if (m < a.m) {
-                    float *y = p.y + (size_t)m * p.ldy + n;
-                    const float v = axq_act(p.act, acc[i][j][r] + bias, a.parts.cap);
-                    *y = p.add ? *y + v : v;
-                }
+                if (m < m1) finish(p, a.parts.cap, m, n, axq_gelu_tanh(acc[i][0][r]) * acc[i][NT - 1][r], true);
             }
+        return;
+    }
+#pragma unroll
+    for (int j = 0; j < NT; j++) {
+        const int n = n0 + wn * (BN / 2) + j * 32 + li;
+        if (n >= p.n) continue;
+#pragma unroll
+        for (int i = 0; i < MT; i++)
+#pragma unroll
+            for (int r = 0; r < 16; r++) {
+                const int m = m0 + wm * (BM / 2) + i * 32 + acc_row(r, lane);
+                if (m < m1) finish(p, a.parts.cap, m, n, acc[i][j][r]);
+            }
+    }
+    if (!GROUPED && p.avg.out) {
+#pragma clang loop unroll(disable)
+        for (int x = 0; x < NT * MT * 16; x++) {
+            const int n = n0 + wn * (BN / 2) + (x & (NT - 1)) * 32 + li, m = m0 + wm * (BM / 2) + x / (NT * 16) * 32 + acc_row((x / NT) & 15, lane);
+            if (n < p.n && m < m1) finish_mean(p, m, n);
+        }
     }
 }
 
 // GEMM on f32 rows in true 32-bit: 64 x 64 tiles, 4 x 4 results per thread, K in steps of 16.
+template <bool GROUPED>
 __global__ void __launch_bounds__(256) dense_gemm_f32_kernel(GemmArgs a) {
     __shared__ __attribute__((aligned(16))) float as[16][68], bs[16][68];
     const int tid = threadIdx.x, tx = tid & 15, ty = tid >> 4;
-    const int tile = xcd_tile(a.tiles), ct = tile / a.mt, m0 = (tile - ct * a.mt) * 64;
-    int pi = 0;
-    while (pi + 1 < a.parts.n_parts && ct >= a.parts.p[pi + 1].blk0) pi++;
+    const int tile = xcd_tile(a.tiles), ct = tile / a.mt;
+    int m0 = (tile - ct * a.mt) * 64, m1 = a.m, pi = 0;
+    size_t woff = 0;
+    if (GROUPED && !group_tile(a.g, tile - ct * a.mt, m0, m1, woff)) return;
+    while (!GROUPED && pi + 1 < a.parts.n_parts && ct >= a.parts.p[pi + 1].blk0) pi++;
     const axq_part &p = a.parts.p[pi];
     const int n0 = (ct - p.blk0) * 64;
     const float *x = reinterpret_cast<const float *>(p.x);
     const int lr = tid >> 2, lc = (tid & 3) * 4; // this thread's four elements of a step: row lr, columns lc ..
-    const float *ga = x + (size_t)(m0 + lr < a.m ? m0 + lr : a.m - 1) * a.ldx + lc;
-    const uint16_t *gb = p.w + (size_t)(n0 + lr < p.n ? n0 + lr : p.n - 1) * p.ldw + lc;
+    int row = m0 + lr < m1 ? m0 + lr : m1 - 1;
+    if (GROUPED && a.g.src) row = a.g.src[row];
+    const float *ga = x + (size_t)row * a.ldx + lc;
+    const uint16_t *gb = p.w + woff + (size_t)(n0 + lr < p.n ? n0 + lr : p.n - 1) * p.ldw + lc;
     float acc[4][4];
 #pragma unroll
     for (int i = 0; i < 4; i++)
@@ -349,10 +467,10 @@ __global__ void __launch_bounds__(256) dense_gemm_f32_kernel(GemmArgs a) {
 #pragma unroll
         for (int j = 0; j < 4; j++) {
             const int m = m0 + ty * 4 + i, n = n0 + tx * 4 + j;
-            if (m < a.m && n < p.n) {
-                float *y = p.y + (size_t)m * p.ldy + n;
-                const float v = axq_act(p.act, acc[i][j] + (p.bias ? p.bias[n] : 0.f), a.parts.cap);
-                *y = p.add ? *y + v : v;
+            if (m < m1 && n < p.n) {
+                const bool glu = p.act == AXQ_ACT_GLU_GELU;
+                finish(p, a.parts.cap, m, n, glu && !(n & AXQ_GLU_GROUP) ? axq_gelu_tanh(acc[i][j]) : acc[i][j], glu);
+                if (!GROUPED && p.avg.out) finish_mean(p, m, n);
             }
         }
 }
@@ -446,6 +564,33 @@ __global__ void __launch_bounds__(256) rows_poly_norm_kernel(axq_in in, axq_rows
     }
 }
 
+__global__ void __launch_bounds__(256) rows_layer_norm_kernel(axq_in in, const float *nw1, axq_rows_out out1, const float *nw2, axq_rows_out out2) {
+    __shared__ float scratch[16];
+    const int t = blockIdx.x, k = in.k;
+    const float *x = in.x + (size_t)(in.rows ? in.rows[t] : t) * k;
+    float sum = 0.f, ss = 0.f;
+    for (int e = threadIdx.x; e < k; e += 256) sum += x[e];
+    const float mean = axq_block_sum(sum, scratch) / (float)k;
+    for (int e = threadIdx.x; e < k; e += 256) {
+        const float d = x[e] - mean;
+        ss = fmaf(d, d, ss);
+    }
+    const float inv = 1.0f / sqrtf(axq_block_sum(ss, scratch) / (float)k + in.eps);
+    for (int e = threadIdx.x; e < out1.ldx; e += 256) {
+        const float n = e < k ? (x[e] - mean) * inv : 0.f;
+        put(out1, t, e, e < k ? n * nw1[e] : 0.f);
+        if (nw2) put(out2, t, e, e < k ? n * nw2[e] : 0.f);
+    }
+}
+
+__global__ void __launch_bounds__(256) rows_glu_kernel(const float *z, int ldz, int k, axq_rows_out out) {
+    const float *row = z + (size_t)blockIdx.x * ldz;
+    for (int e = threadIdx.x; e < out.ldx; e += 256) {
+        const float *g = row + (e / AXQ_GLU_GROUP) * 2 * AXQ_GLU_GROUP + e % AXQ_GLU_GROUP;
+        put(out, blockIdx.x, e, e < k ? g[0] * g[AXQ_GLU_GROUP] : 0.f);
+    }
+}
+
 __global__ void __launch_bounds__(64) rows_zero_tail_kernel(int k, axq_rows_out out) {
     for (int e = k + threadIdx.x; e < out.ldx; e += 64) put(out, blockIdx.x, e, 0.f);
 }
@@ -453,19 +598,35 @@ __global__ void __launch_bounds__(64) rows_zero_tail_kernel(int k, axq_rows_out 
 } // namespace
 
 int axq_dense_gemv(axq_ctx *ctx, int mode, const axq_in &in, axq_parts &parts) {
-    if (in.k < 1 || in.k > AXQ_DENSE_MAX_K || parts.n_parts < 1 || parts.n_parts > AXQ_MAX_PARTS)
+    if ((mode != AXQ_IN_SEGMENTS && (in.k < 1 || in.k > AXQ_DENSE_MAX_K)) || parts.n_parts < 1 || parts.n_parts > AXQ_MAX_PARTS)
         return axq_fail(ctx, AXQ_ERR_SHAPE_MISMATCH, "Shape mismatch: a decode product takes 1 to %d inputs and 1 to %d weights, got %d and %d",
                         AXQ_DENSE_MAX_K, AXQ_MAX_PARTS, in.k, parts.n_parts);
     GemvArgs a;
     a.parts = parts;
     a.in = in;
     a.steps = (in.k + 511) / 512;
+    if (mode == AXQ_IN_SEGMENTS) {
+        a.steps = 0;
+        int items = 0;
+        for (int i = 0; i < in.n_seg; i++) {
+            axq_seg &g = a.in.seg[i];
+            if (g.k < 1 || g.count < 1) return axq_fail(ctx, AXQ_ERR_SHAPE_MISMATCH, "Shape mismatch: segment %d of %d x %d elements", i, g.count, g.k);
+            g.step0 = a.steps;
+            g.steps = (g.k + 511) / 512;
+            a.steps += g.count * g.steps;
+            items += g.count;
+        }
+        if (in.n_seg < 1 || in.n_seg > AXQ_MAX_SEGS || items > AXQ_MAX_SEG_ITEMS || a.steps > AXQ_DENSE_MAX_K / 512 || parts.n_parts != 1)
+            return axq_fail(ctx, AXQ_ERR_SHAPE_MISMATCH, "Shape mismatch: a decode product over %d steps of 512 (at most %d)", a.steps, AXQ_DENSE_MAX_K / 512);
+    }
     switch (mode) {
     case AXQ_IN_PLAIN: return launch_gemv_mode<AXQ_IN_PLAIN>(ctx, a);
     case AXQ_IN_TANH_NORM: return launch_gemv_mode<AXQ_IN_TANH_NORM>(ctx, a);
     case AXQ_IN_TANH_NORM_MIX: return launch_gemv_mode<AXQ_IN_TANH_NORM_MIX>(ctx, a);
     case AXQ_IN_RMS_GATE: return launch_gemv_mode<AXQ_IN_RMS_GATE>(ctx, a);
     case AXQ_IN_POLY_NORM: return launch_gemv_mode<AXQ_IN_POLY_NORM>(ctx, a);
+    case AXQ_IN_LAYER_NORM: return launch_gemv_mode<AXQ_IN_LAYER_NORM>(ctx, a);
+    case AXQ_IN_SEGMENTS: return launch_gemv_mode<AXQ_IN_SEGMENTS>(ctx, a);
     default: return axq_fail(ctx, AXQ_ERR_INVALID_ARGUMENT, "axq_dense_gemv: unknown input mode %d", mode);
     }
 }
@@ -495,16 +656,44 @@ int axq_dense_gemm(axq_ctx *ctx, axq_parts &parts, int m, int k, int ldx, bool f
     for (int i = 0; i < parts.n_parts; i++)
         if (parts.p[i].ldw < a.k || parts.p[i].n < 1)
             return axq_fail(ctx, AXQ_ERR_SHAPE_MISMATCH, "Shape mismatch: weight %d has rows of %d elements, %d wanted", i, parts.p[i].ldw, a.k);
+    bool glu = false;
+    for (int i = 0; i < parts.n_parts; i++) glu |= parts.p[i].act == AXQ_ACT_GLU_GELU;
     if (f32) {
         count_tiles(a, 64, 64);
-        dense_gemm_f32_kernel<<<a.tiles, 256, 0, ctx->stream>>>(a);
+        dense_gemm_f32_kernel<false><<<a.tiles, 256, 0, ctx->stream>>>(a);
     } else if (m > 64 && count_tiles(a, 128, 128) >= ctx->prop.multiProcessorCount) {
-        dense_gemm_kernel<128, 128><<<a.tiles, 256, 0, ctx->stream>>>(a);
+        dense_gemm_kernel<128, 128, false><<<a.tiles, 256, 0, ctx->stream>>>(a);
+    } else if (glu) {
+        count_tiles(a, 64, 128);
+        dense_gemm_kernel<64, 128, false><<<a.tiles, 256, 0, ctx->stream>>>(a);
     } else {
         count_tiles(a, 64, 64);
-        dense_gemm_kernel<64, 64><<<a.tiles, 256, 0, ctx->stream>>>(a);
+        dense_gemm_kernel<64, 64, false><<<a.tiles, 256, 0, ctx->stream>>>(a);
     }
     AXQ_LAUNCH_CHECK(ctx, "dense_gemm_kernel");
+    return AXQ_OK;
+}
+
+int axq_dense_gemm_rows_per_tile(int rows, int groups, bool f32) { return !f32 && rows >= 96 * groups ? 128 : 64; }
+
+int axq_dense_gemm_grouped(axq_ctx *ctx, axq_part &part, const axq_groups &g, int k, int ldx, bool f32) {
+    GemmArgs a;
+    a.parts = {};
+    a.parts.p[0] = part;
+    a.parts.n_parts = 1;
+    a.m = 0;
+    a.k = (k + 63) / 64 * 64;
+    a.ldx = ldx;
+    a.g = g;
+    if (k < 1 || ldx % 64 != 0 || ldx < a.k || part.ldw < a.k || part.n < 1 || g.max_tiles < 1 || (g.bm != 64 && g.bm != 128))
+        return axq_fail(ctx, AXQ_ERR_SHAPE_MISMATCH, "Shape mismatch: grouped rows of %d elements (%d apart) against rows of %d", k, ldx, part.ldw);
+    const int bn = f32 ? 64 : (g.bm == 128 ? 128 : 64);
+    a.mt = g.max_tiles;
+    a.tiles = (part.n + bn - 1) / bn * a.mt;
+    if (f32) dense_gemm_f32_kernel<true><<<a.tiles, 256, 0, ctx->stream>>>(a);
+    else if (g.bm == 128) dense_gemm_kernel<128, 128, true><<<a.tiles, 256, 0, ctx->stream>>>(a);
+    else dense_gemm_kernel<64, 64, true><<<a.tiles, 256, 0, ctx->stream>>>(a);
+    AXQ_LAUNCH_CHECK(ctx, "grouped dense_gemm_kernel");
     return AXQ_OK;
 }
 
@@ -538,6 +727,19 @@ int axq_rows_rms_gate(axq_ctx *ctx, const axq_in &in, int m, int group, axq_rows
 int axq_rows_poly_norm(axq_ctx *ctx, const axq_in &in, int m, axq_rows_out out) {
     rows_poly_norm_kernel<<<m, 256, 0, ctx->stream>>>(in, out);
     AXQ_LAUNCH_CHECK(ctx, "rows_poly_norm_kernel");
+    return AXQ_OK;
+}
+
+int axq_rows_layer_norm(axq_ctx *ctx, const axq_in &in, int m, const float *nw1, axq_rows_out out1, const float *nw2, axq_rows_out out2) {
+    if (nw2 && out2.ldx != out1.ldx) return axq_fail(ctx, AXQ_ERR_SHAPE_MISMATCH, "Shape mismatch: layer norms of rows %d and %d apart", out1.ldx, out2.ldx);
+    rows_layer_norm_kernel<<<m, 256, 0, ctx->stream>>>(in, nw1, out1, nw2, out2);
+    AXQ_LAUNCH_CHECK(ctx, "rows_layer_norm_kernel");
+    return AXQ_OK;
+}
+
+int axq_rows_glu(axq_ctx *ctx, const float *z, int ldz, int k, int m, axq_rows_out out) {
+    rows_glu_kernel<<<m, 256, 0, ctx->stream>>>(z, ldz, k, out);
+    AXQ_LAUNCH_CHECK(ctx, "rows_glu_kernel");
     return AXQ_OK;
 }
 

@@ -9,7 +9,7 @@ import numpy as np
 
 from .hf_loader import HFLoader, UnsupportedFormat, WeightNotFound, set_embedding
 from .quant import ShapeMismatch
-from .stack import ATTENTION, LIGHTNING, WKV, LayerDescription, StackDescription, StackModel
+from .stack import ATTENTION, LIGHTNING, WKV, LayerDescription, StackDescription, StackModel, bench_beside, bench_rates
 
 _NORM = ("", ".b", ".alpha")
 _MIXER_TENSORS = {
@@ -114,25 +114,7 @@ def linear_weights(d):
     return total
 
 
-def _rates(model, weights, bytes_per_weight, prompt, new_tokens):
-    model.generate(prompt, 4)
-    model.reset()
-    pre, dec = [], []
-    for _ in range(3):
-        _, p, d = model.generate(prompt, new_tokens)
-        model.reset()
-        pre.append(p)
-        dec.append(d)
-    pre_ms, dec_ms = sorted(pre)[1], sorted(dec)[1]
-    tok_s = (new_tokens - 1) / (dec_ms * 1e-3)
-    return {"prefill_tokens_per_s": len(prompt) / (pre_ms * 1e-3), "prefill_tflops": 2.0 * weights * len(prompt) / (pre_ms * 1e-3) / 1e12,
-            "decode_tokens_per_s": tok_s, "decode_ms_per_token": 1e3 / tok_s, "decode_weight_gbps": weights * bytes_per_weight * tok_s / 1e9}
-
-
 def bench(ctx, log=print, widths=(1024, 2048, 4096), blocks=2, prompt_len=2048, new_tokens=128, beside=True):
-    from .decode import QuantizedLlama
-    from .quant import QuantType
-
     out = []
     for width in widths:
         d = bench_description(width, blocks, prompt_len + new_tokens)
@@ -141,22 +123,10 @@ def bench(ctx, log=print, widths=(1024, 2048, 4096), blocks=2, prompt_len=2048, 
         m = StackModel(d, ctx=ctx)
         m.random_init(0.02, 1)
         r = {"width": width, "layers": len(d.layers), "linear_weights": weights, "prompt_tokens": prompt_len, "generated_tokens": new_tokens,
-             "lakulix_bf16": _rates(m, weights, 2.0, prompt, new_tokens)}
+             "lakulix_bf16": bench_rates(m, weights, 2.0, prompt, new_tokens)}
         m.close()
         if beside:
-            heads, ff = width // 128, width * 7 // 2
-            kv = max(1, heads // 4)
-            per_layer = width * (2 * width + 2 * kv * 128 + 3 * ff)
-            n = max(1, round((weights - d.vocab_size * width) / per_layer))
-            cfg = dict(vocab_size=d.vocab_size, hidden_size=width, intermediate_size=ff, num_hidden_layers=n, num_attention_heads=heads,
-                       num_key_value_heads=kv, head_dim=128, max_position_embeddings=prompt_len + new_tokens, rms_norm_eps=1e-5,
-                       rope_theta=10000.0)
-            lw = n * per_layer + d.vocab_size * width
-            for qt, bpw in ((QuantType.BF16, 2.0), (QuantType.Q4_K, 0.5625)):
-                lm = QuantizedLlama(ctx, **cfg)
-                lm.random_init(qt, 0.02, 1)
-                r[f"llama_{str(qt).lower()}"] = dict(_rates(lm, lw, bpw, prompt, new_tokens), layers=n, linear_weights=lw)
-                lm.close()
+            r.update(bench_beside(ctx, width, weights, d.vocab_size, prompt, new_tokens))
         for name, v in r.items():
             if isinstance(v, dict):
                 log(f"  width {width} {name}: prefill {v['prefill_tokens_per_s']:.0f} tok/s ({v['prefill_tflops']:.0f} TFLOP/s), decode "

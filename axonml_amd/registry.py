@@ -51,3 +51,12 @@ def _lakulix(path, dtype, max_positions, quant_type, ctx):
     if quant_type not in (None, QuantType.BF16):
         raise UnsupportedFormat(f"Lakulix linears are kept in BF16, not {QuantType(quant_type)}")
     return load(path, dtype, max_positions, ctx)
+
+
+@register("Gemosun")
+def _gemosun(path, dtype, max_positions, quant_type, ctx):
+    from .gemosun import load
+
+    if quant_type not in (None, QuantType.BF16):
+        raise UnsupportedFormat(f"Gemosun linears are kept in BF16, not {QuantType(quant_type)}")
+    return load(path, dtype, max_positions, ctx)

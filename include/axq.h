@@ -287,19 +287,42 @@ typedef enum {
                               per-head RMS norms on q and k; q times 1 + q_temp_coef ln(floor((p + 1) / q_temp_every) + 1);
                               score = q.k * scale + learned bias by distance (bias_rows buckets up to bias_max) */
     AXQ_MIX_LIGHTNING = 1, /* linear attention: S <- decay S + k v^T, o = S^T q; SiLU on q, k, v; gated RMS norm over all heads */
-    AXQ_MIX_WKV = 2        /* time mixing: inputs leaning to the previous token's, a decay per token, head and key channel
+    AXQ_MIX_WKV = 2,       /* time mixing: inputs leaning to the previous token's, a decay per token, head and key channel
                               (through decay_rank), a bonus for the current token, gated RMS norm per head */
+    AXQ_MIX_SOFTMAX = 3    /* causal softmax attention, score = q.k * scale, over the last `window` tokens and, with `pool` P, over
+                              one key and value per block of P tokens that lies wholly before the window, the means of its
+                              tokens'; rotary positions on the first rot_dims dimensions of q and k (neighbours paired);
+                              keys_as_values: values are the keys before rotation, there is no "mix.v"; head_gate: each
+                              head's result times sigmoid of a product of its own, "mix.g" */
 } axq_mixer;
-/* Norms are tanh(alpha x) w + b.  Feed-forward (ff > 0): W_down act(W_up n(x)), act(z) = a N(z) + b N(z^2) + c N(z^3) + e with
- * N(z) = z / sqrt(mean(z^2) + eps). */
+/* Feed-forwards, of h = norm2(x) (ff > 0). */
+typedef enum {
+    AXQ_FF_POLY = 0,  /* down act(up h), act(z) = a N(z) + b N(z^2) + c N(z^3) + e, N(z) = z / sqrt(mean(z^2) + eps) */
+    AXQ_FF_GLU = 1,   /* down (gelu_tanh(gate h) * up h) */
+    AXQ_FF_MOE = 2    /* experts e: down_e relu(up_e h)^2; a token goes through the `top` of `experts` with the best scores
+                         sigmoid(router h) among those of the groups_keep best of `groups` equal groups of neighbours (by the sum of
+                         their two best scores), weighted by score / sum of the chosen ones; shared_ff > 0: and one such
+                         expert for every token, times sigmoid(shared.sg h) */
+} axq_ff_kind;
+typedef enum {
+    AXQ_NORM_TANH = 0, /* tanh(alpha x) w + b */
+    AXQ_NORM_LAYER = 1 /* (x - mean) / sqrt(mean((x - mean)^2) + eps) w */
+} axq_norm_kind;
+/* What a layer does not use is 0. */
 typedef struct {
     int32_t mixer;                          /* axq_mixer */
-    int32_t heads, kv_heads, dim, vdim;     /* kv_heads: attention only; wkv: vdim = dim */
-    int32_t ff;                             /* 0: no feed-forward sublayer */
+    int32_t heads, kv_heads, dim, vdim;     /* kv_heads: attentions only; wkv: vdim = dim */
+    int32_t ff;                             /* width of the feed-forward, or of one expert; 0: no feed-forward */
     int32_t bias_rows, bias_max;            /* attention; bias_rows 0: no distance bias */
     int32_t q_temp_every;                   /* attention; 0: no query factor */
-    float q_temp_coef, scale;               /* attention */
+    float q_temp_coef, scale;               /* attention; scale: both attentions */
     int32_t decay_rank;                     /* wkv */
+    int32_t window, pool;                   /* softmax attention; window 0: all tokens; pool 0: no blocks */
+    int32_t keys_as_values, head_gate;      /* softmax attention, 0 or 1 */
+    int32_t rot_dims, rot_original;         /* softmax attention; rot_dims 0: no rotation; rot_original 0: no scaling (YaRN) */
+    double rot_base, rot_factor, rot_fast, rot_slow;
+    int32_t ff_kind;                        /* axq_ff_kind */
+    int32_t experts, top, groups, groups_keep, shared_ff; /* AXQ_FF_MOE */
 } axq_layer_config;
 typedef enum { AXQ_COMPUTE_BF16 = 0, AXQ_COMPUTE_F32 = 1 } axq_compute;
 typedef struct {
@@ -312,11 +335,18 @@ typedef struct {
     float norm_eps;
     float logit_softcap;                    /* logits <- cap tanh(logits / cap); 0: none */
     const axq_layer_config *layers;         /* num_layers */
+    int32_t norm;                           /* axq_norm_kind, of all norms of the residual stream */
+    int32_t position_table;                 /* 1: "pos" is added to the embedding */
+    int32_t parallel;                       /* 1: x + (mixer(norm1(x)) + ff(norm2(x))) instead of one after the other (layer norms only) */
+    int32_t depth_average;                  /* 1: after layer i, x <- sum over j <= i + 1 of "dwa"[j] X_j: X_0 the embedding, X_(j+1) layer
+                                               j's result before this (no loop) */
 } axq_stack_config;
 AXQ_API int axq_model_create_stack(axq_ctx *ctx, const axq_stack_config *cfg, axq_model **out);
-/* A tensor by name, from f32 values (host): layer -1 = "pos" [max_positions, width], "final.norm", "final.norm.b" [width],
- * "final.norm.alpha" [1], "head" [vocab, width]; a layer's "norm1", "norm1.b", "norm1.alpha", "norm2" likewise, its mixer's
- * "mix.q" ..., its feed-forward's "mlp.up", "mlp.down", "mlp.act" [4].  Linears ([out, in]) are kept as AXQ_BF16.  rows x cols
+/* A tensor by name, from f32 values (host): layer -1 = "pos" [max_positions, width], "final.norm" [width] (tanh norm: and
+ * "final.norm.b" [width], "final.norm.alpha" [1]), "head" [vocab, width]; a layer's "norm1" and "norm2" likewise, its mixer's
+ * "mix.q" ..., "dwa" [layer + 2], its feed-forward's "mlp.up", "mlp.down", "mlp.act" [4] (poly), "mlp.gate", "mlp.up",
+ * "mlp.down" (glu), "mlp.router" [experts, width], "mlp.e<i>.up", "mlp.e<i>.down", "mlp.shared.up", "mlp.shared.down",
+ * "mlp.shared.sg" [1, width] (moe).  Linears ([out, in]) are kept as AXQ_BF16.  rows x cols
  * must be the tensor's shape (rows = 1 for vectors).  The embedding goes through axq_model_set_embedding_f32 / _f16. */
 AXQ_API int axq_model_set_tensor(axq_model *m, int layer, const char *name, const float *data, int64_t rows, int64_t cols);
 

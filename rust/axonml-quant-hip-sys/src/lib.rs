@@ -24,6 +24,9 @@ pub struct axq_model_config {
 pub struct axq_layer_config {
     pub mixer: i32, pub heads: i32, pub kv_heads: i32, pub dim: i32, pub vdim: i32, pub ff: i32,
     pub bias_rows: i32, pub bias_max: i32, pub q_temp_every: i32, pub q_temp_coef: f32, pub scale: f32, pub decay_rank: i32,
+    pub window: i32, pub pool: i32, pub keys_as_values: i32, pub head_gate: i32, pub rot_dims: i32, pub rot_original: i32,
+    pub rot_base: f64, pub rot_factor: f64, pub rot_fast: f64, pub rot_slow: f64,
+    pub ff_kind: i32, pub experts: i32, pub top: i32, pub groups: i32, pub groups_keep: i32, pub shared_ff: i32,
 }
 
 #[repr(C)]
@@ -31,6 +34,7 @@ pub struct axq_stack_config {
     pub vocab_size: i32, pub width: i32, pub max_positions: i32, pub cache_positions: i32, pub num_layers: i32,
     pub loop_start: i32, pub loop_stop: i32, pub loop_times: i32, pub compute: i32, pub norm_eps: f32, pub logit_softcap: f32,
     pub layers: *const axq_layer_config,
+    pub norm: i32, pub position_table: i32, pub parallel: i32, pub depth_average: i32,
 }
 
 #[link(name = "axq")]
