@@ -66,7 +66,7 @@ struct axq_stack {
     std::vector<Rotation> rotations;
     // activations of a step
     float *proj = nullptr, *o = nullptr, *z = nullptr, *part = nullptr;
-    float *past = nullptr; // depth average: the embedding and every layer's result
+    float *past = nullptr; // mean over the layers: the embedding and every layer's result
     float *ez = nullptr, *wt = nullptr; // mixture: the chosen experts' inner activations and weights
     int32_t *sel = nullptr;
     void *qs = nullptr;
@@ -76,7 +76,7 @@ struct axq_stack {
     float *r_seg = nullptr, *r_segw = nullptr; // segments of a recurrence
     void *r_x = nullptr, *r_qs = nullptr;
     void *r_x2 = nullptr, *r_f = nullptr; // operands: the second norm of a parallel layer; what goes into a feed-forward's last product
-    float *r_past = nullptr;              // depth average
+    float *r_past = nullptr;              // mean over the layers
     void *r_ez = nullptr;                 // mixture: by slot, the operands of the experts' last products,
     float *r_ey = nullptr, *r_wt = nullptr; // ... their results; by row, the weights
     int32_t *r_route = nullptr;           // ... and the chosen experts, slots, rows by slot and tiles
@@ -567,7 +567,7 @@ int axq_stack_step(axq_model *m) {
         axq_in in = norm_in(s, l, "norm1", x), out_in;
         Proj p;
         add_firsts(p, l, mixer_firsts(c), s.proj, 1, in.nw);
-        float *const *ff = p.out.data() + p.out.size();
+        float *const *ff = nullptr;
         if (parallel) {
             p.out.reserve(p.out.size() + 8);
             ff = p.out.data() + p.out.size();

@@ -411,6 +411,9 @@ def main():
                          "models of equal size, as one JSON line")
     ap.add_argument("--lakulix-widths", default="1024,2048,4096", help="widths of --lakulix")
     ap.add_argument("--lakulix-only", action="store_true", help="with --lakulix, for kernel profiles: without the LLaMA-shape models")
+    ap.add_argument("--gemosun", action="store_true", help="the same for Gemosun models")
+    ap.add_argument("--gemosun-widths", default="1024,2048,4096", help="widths of --gemosun")
+    ap.add_argument("--gemosun-only", action="store_true", help="with --gemosun, for kernel profiles: without the LLaMA-shape models")
     ap.add_argument("--grid-barrier", action="store_true",
                     help="instead of the benchmark: time a barrier over all workgroups of one resident launch through device-scope "
                          "atomics (what a kernel that spans dependent steps would pay per step), and print the table")
@@ -446,6 +449,13 @@ def main():
 
         res = lakulix.bench(ctx, log, widths=tuple(int(w) for w in args.lakulix_widths.split(",")), beside=not args.lakulix_only)
         print(json.dumps({"lakulix": res}), flush=True)
+        ctx.close()
+        return
+    if args.gemosun or args.gemosun_only:
+        from axonml_amd import gemosun
+
+        res = gemosun.bench(ctx, log, widths=tuple(int(w) for w in args.gemosun_widths.split(",")), beside=not args.gemosun_only)
+        print(json.dumps({"gemosun": res}), flush=True)
         ctx.close()
         return
     if args.gemv_table:

@@ -1,18 +1,9 @@
 """Random Lakulix models for the tests: configurations as config.json spells them and weights as plain arrays, bfloat16
 exact, for the product (`axonml_amd.lakulix.build`) and for the plain forward (`oracle.lakulix.Model`) alike."""
-import json
-import os
-import struct
-
 import numpy as np
 
+from .stack_common import LIMIT, bf16, error, write_checkpoint  # noqa: F401
 from oracle import lakulix as plain
-
-
-def bf16(x):
-    """Rounded to bfloat16 (nearest even), as f32."""
-    u = np.ascontiguousarray(x, dtype=np.float32).view(np.uint32).astype(np.uint64)
-    return (((u + 0x7FFF + ((u >> 16) & 1)) >> 16) << 16).astype(np.uint32).view(np.float32).reshape(np.shape(x))
 
 
 def attention(heads=4, kv_heads=2, dim=24, vdim=16, ff=0, bias_max=40, scale=0.2, coef=0.4, every=9):
@@ -96,31 +87,3 @@ def product(cfg, t, dtype, ctx, cache_positions=None):
     from axonml_amd import lakulix
 
     return lakulix.build(cfg, lambda n: t[n], lambda n: list(t[n].shape) if n in t else None, dtype, cache_positions, ctx)
-
-
-def error(got, want):
-    """Per position: rms of the difference over the vocabulary (mean taken off), relative to the typical spread of the logits."""
-    got, want = np.asarray(got, np.float64), np.asarray(want, np.float64)
-    d = got - want
-    d -= d.mean(-1, keepdims=True)
-    scale = np.sqrt(np.mean((want - want.mean(-1, keepdims=True)) ** 2))
-    return np.sqrt((d * d).mean(-1)) / scale
-
-
-# f32: accumulation noise of a few layers over some hundred terms.  bf16: rounding of the products' inputs to 8 bits.
-LIMIT = {"float32": 2e-5, "bfloat16": 3e-2}
-
-
-def write_checkpoint(path, cfg, t):
-    """config.json and model.safetensors (bfloat16) in the directory `path`."""
-    with open(os.path.join(path, "config.json"), "w") as f:
-        json.dump(cfg, f)
-    header, blobs, at = {}, [], 0
-    for name, a in t.items():
-        b = (np.ascontiguousarray(a, np.float32).view(np.uint32) >> 16).astype("<u2").tobytes()
-        header[name] = {"dtype": "BF16", "shape": list(np.shape(a)), "data_offsets": [at, at + len(b)]}
-        blobs.append(b)
-        at += len(b)
-    head = json.dumps(header).encode()
-    with open(os.path.join(path, "model.safetensors"), "wb") as f:
-        f.write(struct.pack("<Q", len(head)) + head + b"".join(blobs))

@@ -9,6 +9,7 @@ import numpy as np
 import pytest
 
 from . import lakulix_common as lc
+from .stack_common import close, feed, tokens_of
 from oracle import lakulix as plain
 
 pytestmark = pytest.mark.gpu
@@ -44,27 +45,6 @@ ONE_LAYER = {
     "feed-forward": (lc.config([lc.lightning(heads=1, dim=4, vdim=4, ff=200)]), {}),
     "feed-forward narrow": (lc.config([lc.wkv(heads=1, dim=8, ff=3)]), {}),
 }
-
-
-def tokens_of(cfg, n, seed=5):
-    return np.random.default_rng(seed).integers(0, cfg["vocab"], n)
-
-
-def close(got, want, dtype, layers=1):
-    """f32: every position.  bfloat16: nearly all of them, and none far off (sums over many keys can nearly cancel, and then a
-    position answers to rounding with several times the usual error)."""
-    e, limit = lc.error(got, want), lc.LIMIT[dtype] * layers
-    return e.max() < limit if dtype == "float32" else np.quantile(e, 0.97) < limit and e.max() < 3 * limit
-
-
-def feed(model, tokens, cuts):
-    """All logits, the tokens cut into portions."""
-    at, out = 0, []
-    for n in cuts:
-        out.append(model.feed(tokens[at:at + n], list(range(n))))
-        at += n
-    assert at == len(tokens)
-    return np.concatenate(out)
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
