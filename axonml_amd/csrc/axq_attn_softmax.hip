@@ -1,6 +1,6 @@
 // Causal softmax attention over a sliding window of tokens and, where asked for, the means of blocks of older tokens:
-// position i sees tokens i - window + 1 .. i and block b (tokens bP .. bP + P - 1) once (b + 1) P <= i - window + 1, as one key
-// and one value, the means of the cached ones.  Queries and keys may be rotated in part (neighbouring dimensions), values may
+// with s = max(0, p - window + 1), position p sees the tokens s .. p and the first s / pool blocks of `pool` tokens, each as one
+// key and one value, the means of the cached ones (what lies between the last whole block and s is not seen).  Queries and keys may be rotated in part (neighbouring dimensions), values may
 // be the keys before rotation, each head's result may be gated.
 //
 // The blocks' keys and values are a second cache of the same layout (axq_attn_tiles.h); all kernels walk the blocks first and
@@ -33,12 +33,13 @@ __device__ inline float rotated(const axq_soft_attn &a, const float *x, int e, i
     return (e & 1) ? fmaf(v, c, w * s) : fmaf(v, c, -(w * s));
 }
 
-// grid (heads + kv_heads (+ kv_heads of values in f32), rows), one wave: rotated queries, keys into the cache
+// grid (heads + kv_heads (+ kv_heads of values in f32) in fours, rows), a wave each: rotated queries, keys into the cache
 template <bool F32>
-__global__ void __launch_bounds__(64) prep_kernel(Args g) {
+__global__ void __launch_bounds__(256) prep_kernel(Args g) {
     const axq_soft_attn &a = g.a;
-    const int t = blockIdx.y, lane = threadIdx.x, p = g.pos ? g.pos[0] : g.pos0 + t;
-    int h = blockIdx.x;
+    const int t = blockIdx.y, lane = threadIdx.x & 63, p = g.pos ? g.pos[0] : g.pos0 + t;
+    int h = blockIdx.x * 4 + (threadIdx.x >> 6);
+    if (h >= a.heads + (F32 ? 2 : 1) * a.kv_heads) return;
     if (h < a.heads) {
         const float *q = g.q + (size_t)t * g.ldq + (size_t)h * a.dim;
         if (F32) {
@@ -83,14 +84,17 @@ __device__ void pool_block(const Args &g, int h, int b, int tid, int n) {
         if (F32) {
             const int d = key ? a.dim : a.vdim;
             const float *x = reinterpret_cast<const float *>(key ? a.kc : a.vc) + ((size_t)h * a.cap + p0) * d + e;
+#pragma unroll 16
             for (int j = 0; j < a.pool; j++) s += x[(size_t)j * d];
             reinterpret_cast<float *>(key ? a.pkc : a.pvc)[((size_t)h * g.cap_blocks + b) * d + e] = s * inv;
         } else if (key) {
             const _Float16 *x = reinterpret_cast<const _Float16 *>(a.kc) + ((size_t)h * g.capp + p0) * g.dp + e;
+#pragma unroll 16
             for (int j = 0; j < a.pool; j++) s += (float)x[(size_t)j * g.dp];
             reinterpret_cast<_Float16 *>(a.pkc)[((size_t)h * g.cpp + b) * g.dp + e] = (_Float16)(s * inv);
         } else {
             const _Float16 *x = reinterpret_cast<const _Float16 *>(a.vc) + ((size_t)h * g.dvp + e) * g.capp;
+#pragma unroll 16
             for (int j = 0; j < a.pool; j++) s += (float)x[value_slot((int)p0 + j)];
             reinterpret_cast<_Float16 *>(a.pvc)[((size_t)h * g.dvp + e) * g.cpp + value_slot(b)] = (_Float16)(s * inv);
         }
@@ -99,7 +103,7 @@ __device__ void pool_block(const Args &g, int h, int b, int tid, int n) {
 
 // grid (kv heads, blocks that end within the rows)
 template <bool F32>
-__global__ void __launch_bounds__(128) pool_kernel(Args g) {
+__global__ void __launch_bounds__(256) pool_kernel(Args g) {
     int b;
     if (g.pos) {
         const int n = g.pos[0] + 1;
@@ -108,7 +112,7 @@ __global__ void __launch_bounds__(128) pool_kernel(Args g) {
     } else {
         b = g.pos0 / g.a.pool + blockIdx.y;
     }
-    pool_block<F32>(g, blockIdx.x, b, threadIdx.x, 128);
+    pool_block<F32>(g, blockIdx.x, b, threadIdx.x, 256);
 }
 
 // Rows against the f32 caches: grid (heads, rows).  256 keys at a time: scores by thread, then the value sum by element.
@@ -532,7 +536,7 @@ template <bool F32>
 void launch_pool(axq_ctx *ctx, const Args &g) {
     if (g.a.pool < 1 || g.cap_blocks < 1) return;
     const int n = g.pos ? 1 : (g.pos0 + g.m) / g.a.pool - g.pos0 / g.a.pool;
-    if (n > 0) pool_kernel<F32><<<dim3(g.a.kv_heads, n), 128, 0, ctx->stream>>>(g);
+    if (n > 0) pool_kernel<F32><<<dim3(g.a.kv_heads, n), 256, 0, ctx->stream>>>(g);
 }
 
 } // namespace
@@ -560,11 +564,11 @@ int axq_soft_attn_rows(axq_ctx *ctx, const axq_soft_attn &a, const float *q, con
         return axq_fail(ctx, AXQ_ERR_OVERFLOW, "Numerical overflow during quantization: positions %d .. %d beyond the cache of %d", pos0, pos0 + m, a.cap);
     const Args g = make_args(a, q, k, v, gate, ldq, ldk, ldv, m, pos0, nullptr, qscratch);
     if (a.f32) {
-        prep_kernel<true><<<dim3(a.heads + 2 * a.kv_heads, m), 64, 0, ctx->stream>>>(g);
+        prep_kernel<true><<<dim3((a.heads + 2 * a.kv_heads + 3) / 4, m), 256, 0, ctx->stream>>>(g);
         launch_pool<true>(ctx, g);
         rows_f32_kernel<<<dim3(a.heads, m), 256, f32_rows_lds(a), ctx->stream>>>(g, out);
     } else {
-        prep_kernel<false><<<dim3(a.heads + a.kv_heads, m), 64, 0, ctx->stream>>>(g);
+        prep_kernel<false><<<dim3((a.heads + a.kv_heads + 3) / 4, m), 256, 0, ctx->stream>>>(g);
         append_values_kernel<<<dim3((m + 31) / 32, (a.vdim + 31) / 32, a.kv_heads), 256, 0, ctx->stream>>>(g);
         launch_pool<false>(ctx, g);
         if ((rc = g.dp == 64 ? launch_mfma_k<4>(ctx, g, out) : (g.dp == 128 ? launch_mfma_k<8>(ctx, g, out) : launch_mfma_k<16>(ctx, g, out)))) return rc;
@@ -579,7 +583,7 @@ int axq_soft_attn_token(axq_ctx *ctx, const axq_soft_attn &a, const float *q, co
     if ((rc = check_shape(ctx, a))) return rc;
     const Args g = make_args(a, q, k, v, gate, 0, 0, 0, 1, 0, pos, qscratch);
     if (a.f32) {
-        prep_kernel<true><<<dim3(a.heads + 2 * a.kv_heads, 1), 64, 0, ctx->stream>>>(g);
+        prep_kernel<true><<<dim3((a.heads + 2 * a.kv_heads + 3) / 4, 1), 256, 0, ctx->stream>>>(g);
         launch_pool<true>(ctx, g);
         axq_rows_out out = {att, a.heads * a.vdim, true};
         rows_f32_kernel<<<dim3(a.heads, 1), 256, f32_rows_lds(a), ctx->stream>>>(g, out);

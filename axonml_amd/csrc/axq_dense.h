@@ -162,8 +162,8 @@ int axq_sig_attn_token(axq_ctx *ctx, const axq_sig_attn &a, const float *q, cons
 struct axq_soft_attn {
     int heads, kv_heads, dim, vdim;
     int cap;                 // positions the cache holds
-    int window;              // position i sees tokens i - window + 1 .. i
-    int pool;                // 0: no more; P: and one key and value, the mean of P, for each block bP .. bP + P - 1 with bP + P - 1 <= i - window
+    int window;              // tokens seen, the newest one included
+    int pool;                // tokens of a block that is seen, as its mean key and value, once the window has left it behind; 0: no blocks
     float scale;
     int rot_dims;            // neighbours (2i, 2i + 1) of the first rot_dims dimensions are rotated; 0: none
     const float *rc, *rs;    // [positions][rot_dims / 2] cosines and sines

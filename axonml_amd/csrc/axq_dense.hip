@@ -8,6 +8,8 @@ namespace {
 typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
 typedef float f32x16 __attribute__((ext_vector_type(16)));
 typedef uint32_t u32x4 __attribute__((ext_vector_type(4)));
+typedef float f32x4 __attribute__((ext_vector_type(4)));
+typedef float f32x4_any __attribute__((ext_vector_type(4), aligned(4))); // at any float's address
 typedef const __attribute__((address_space(1))) void gbl_void;
 typedef __attribute__((address_space(3))) void lds_void;
 
@@ -27,47 +29,73 @@ struct GemvArgs {
     int steps; // of 512 elements
 };
 
+// Of a step of AXQ_IN_SEGMENTS: its weight's columns, their row pitch and 16-byte chunks; its inputs, their number and factor.
+struct Step { const uint16_t *w; int ldw, c8; const float *x; float f; int k, glu; };
+
+// Four inputs from e on, zeros past the end
+__device__ inline f32x4 load_quad(const float *x, int e, int k) {
+    if (e + 4 <= k) return *reinterpret_cast<const f32x4_any *>(x + e);
+    f32x4 v = {0.f, 0.f, 0.f, 0.f};
+    for (int i = 0; i < 4; i++)
+        if (e + i < k) v[i] = x[e + i];
+    return v;
+}
+__device__ inline f32x4 load_step(const Step &t, int e) {
+    f32x4 v;
+    if (t.glu) { // both halves are padded to whole groups
+        const float *z = t.x + (e / AXQ_GLU_GROUP) * 2 * AXQ_GLU_GROUP + e % AXQ_GLU_GROUP;
+        v = load_quad(z, 0, t.k - e) * load_quad(z + AXQ_GLU_GROUP, 0, t.k - e);
+    } else {
+        v = load_quad(t.x, e, t.k);
+    }
+    return v * t.f;
+}
+
 template <int MODE>
-__device__ void stage_x(const GemvArgs &a, const axq_part &p, float *xs, float *scratch) {
+__device__ void stage_x(const GemvArgs &a, const axq_part &p, const Step *table, float *xs, float *scratch) {
     const axq_in &in = a.in;
     const float *mu = p.mu;
-    const int k = in.k, tid = threadIdx.x, xl = a.steps * 512, half = xl >> 1;
+    const int k = in.k, tid = threadIdx.x, xl = a.steps * 512, half = xl >> 1, quads = xl >> 2;
     auto slot = [half](int e) { return ((e >> 3) << 2) + (e & 3) + ((e & 4) ? half : 0); };
-    if (MODE == AXQ_IN_SEGMENTS) {
-        for (int s = 0; s < in.n_seg; s++) {
-            const axq_seg &g = in.seg[s];
-            const int span = g.steps * 512;
-            for (int i = 0; i < g.count; i++) {
-                const float *x = g.x + (size_t)i * g.ldx, f = g.scale ? g.scale[i] : 1.0f;
-                const int e0 = (g.step0 + i * g.steps) * 512;
-                for (int e = tid; e < span; e += GT) {
-                    float v = 0.f;
-                    if (e < g.k) {
-                        if (g.glu) {
-                            const float *z = x + (e / AXQ_GLU_GROUP) * 2 * AXQ_GLU_GROUP + e % AXQ_GLU_GROUP;
-                            v = z[0] * z[AXQ_GLU_GROUP];
-                        } else {
-                            v = x[e];
-                        }
-                    }
-                    xs[slot(e0 + e)] = v * f;
-                }
+    auto quad = [half, xs](int q) -> f32x4 & { return *reinterpret_cast<f32x4 *>(xs + ((q >> 1) << 2) + ((q & 1) ? half : 0)); };
+    if (MODE == AXQ_IN_SEGMENTS) { // four loads under way per thread
+        for (int q0 = tid; q0 < quads; q0 += 4 * GT) {
+            f32x4 v[4];
+#pragma unroll
+            for (int i = 0; i < 4; i++) {
+                const int q = q0 + i * GT;
+                if (q < quads) v[i] = load_step(table[q >> 7], (q & 127) << 2);
             }
+#pragma unroll
+            for (int i = 0; i < 4; i++)
+                if (q0 + i * GT < quads) quad(q0 + i * GT) = v[i];
         }
     } else if (MODE == AXQ_IN_LAYER_NORM) {
+        constexpr int NW = 2; // the first quads' weights are requested with the inputs
+        f32x4 w[NW];
         float sum = 0.f, ss = 0.f;
-        for (int e = tid; e < k; e += GT) {
-            const float v = in.x[e];
-            xs[slot(e)] = v;
-            sum += v;
+#pragma unroll
+        for (int i = 0; i < NW; i++)
+            if (tid + i * GT < quads) w[i] = load_quad(p.nw, (tid + i * GT) << 2, k);
+        for (int q = tid; q < quads; q += GT) {
+            const f32x4 v = load_quad(in.x, q << 2, k);
+            quad(q) = v;
+            sum += (v[0] + v[1]) + (v[2] + v[3]);
         }
         const float mean = axq_block_sum(sum, scratch) / (float)k;
-        for (int e = tid; e < k; e += GT) {
-            const float d = xs[slot(e)] - mean;
-            ss = fmaf(d, d, ss);
+        for (int q = tid; q < quads; q += GT) {
+            const f32x4 v = quad(q);
+#pragma unroll
+            for (int i = 0; i < 4; i++) {
+                const float d = (q << 2) + i < k ? v[i] - mean : 0.f;
+                ss = fmaf(d, d, ss);
+            }
         }
         const float inv = 1.0f / sqrtf(axq_block_sum(ss, scratch) / (float)k + in.eps);
-        for (int e = tid; e < xl; e += GT) xs[slot(e)] = e < k ? (xs[slot(e)] - mean) * inv * p.nw[e] : 0.f;
+#pragma unroll
+        for (int i = 0; i < NW; i++)
+            if (tid + i * GT < quads) quad(tid + i * GT) = (quad(tid + i * GT) - mean) * inv * w[i]; // zeros past the end
+        for (int q = tid + NW * GT; q < quads; q += GT) quad(q) = (quad(q) - mean) * inv * load_quad(p.nw, q << 2, k);
     } else
     if (MODE == AXQ_IN_RMS_GATE) {
         float ss = 0.f;
@@ -119,7 +147,6 @@ __global__ void __launch_bounds__(GT, 4) dense_gemv_kernel(GemvArgs a) {
     extern __shared__ __attribute__((aligned(16))) float xs[];
     __shared__ float scratch[16];
     constexpr bool SEG = MODE == AXQ_IN_SEGMENTS;
-    struct Step { const uint16_t *w; int ldw, c8; }; // of a step: its weight's columns, their row pitch and 16-byte chunks
     __shared__ Step table[SEG ? AXQ_DENSE_MAX_K / 512 : 1];
     constexpr int U = 8 / R;
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
@@ -139,6 +166,10 @@ __global__ void __launch_bounds__(GT, 4) dense_gemv_kernel(GemvArgs a) {
             table[t].w = g.w + (size_t)(g.sel ? g.sel[i] : i) * g.stride + (size_t)s * 512;
             table[t].ldw = g.ldw;
             table[t].c8 = ((g.k + 7) >> 3) - s * 64;
+            table[t].x = g.x + (size_t)i * g.ldx + (size_t)s * (g.glu ? 1024 : 512);
+            table[t].f = g.scale ? g.scale[i] : 1.0f;
+            table[t].k = g.k - s * 512;
+            table[t].glu = g.glu;
         }
         __syncthreads();
     }
@@ -152,7 +183,7 @@ __global__ void __launch_bounds__(GT, 4) dense_gemv_kernel(GemvArgs a) {
             if (SEG) {
 #pragma unroll
                 for (int u = 0; u < U; u++) {
-                    const Step t = table[s0 + u < a.steps ? s0 + u : a.steps - 1];
+                    const Step &t = table[s0 + u < a.steps ? s0 + u : a.steps - 1];
                     const int c = lane < t.c8 ? lane : t.c8 - 1;
                     q[u][r] = __builtin_nontemporal_load(reinterpret_cast<const u32x4 *>(t.w + (size_t)row * t.ldw + (size_t)c * 8));
                 }
@@ -183,7 +214,7 @@ __global__ void __launch_bounds__(GT, 4) dense_gemv_kernel(GemvArgs a) {
         if (staged < 0 || (MODE == AXQ_IN_TANH_NORM_MIX && staged != pi) ||
             (MODE == AXQ_IN_LAYER_NORM && a.parts.p[staged].nw != p.nw)) { // the same for all waves
             if (staged >= 0) __syncthreads();
-            stage_x<MODE>(a, p, xs, scratch);
+            stage_x<MODE>(a, p, table, xs, scratch);
             staged = pi;
         }
 #pragma unroll
@@ -249,8 +280,8 @@ int launch_gemv(axq_ctx *ctx, GemvArgs &a) {
         nb += (a.parts.p[i].n + GW * R - 1) / (GW * R);
     }
     a.parts.n_blocks = nb;
-    const int most = 2 * ctx->prop.multiProcessorCount;
     const size_t lds = (size_t)a.steps * 512 * sizeof(float);
+    const int most = (lds > 76 * 1024 ? 1 : 2) * ctx->prop.multiProcessorCount; // as many as are there at once
     static std::atomic<uint64_t> lds_allowed{0};
     int rc;
     if (lds > 48 * 1024 &&
@@ -494,6 +525,13 @@ __device__ inline void put(const axq_rows_out &o, size_t row, int e, float v) {
     else reinterpret_cast<uint16_t *>(o.x)[row * o.ldx + e] = axq_to_bf16(v);
 }
 
+__device__ inline void put_quad(const axq_rows_out &o, size_t row, int e, f32x4 v) { // e and rows: multiples of 4
+    if (o.f32) *reinterpret_cast<f32x4 *>(reinterpret_cast<float *>(o.x) + row * o.ldx + e) = v;
+    else
+        *reinterpret_cast<uint2 *>(reinterpret_cast<uint16_t *>(o.x) + row * o.ldx + e) =
+            make_uint2(axq_to_bf16(v[0]) | (uint32_t)axq_to_bf16(v[1]) << 16, axq_to_bf16(v[2]) | (uint32_t)axq_to_bf16(v[3]) << 16);
+}
+
 __global__ void __launch_bounds__(256) embed_pos_kernel(const uint16_t *emb16, const float *emb32, const float *pos_table, const int32_t *tok,
                                                         const int32_t *pos, int pos0, int width, float *h) {
     const int e = blockIdx.x * 256 + threadIdx.x, t = blockIdx.y;
@@ -566,17 +604,39 @@ __global__ void __launch_bounds__(256) rows_poly_norm_kernel(axq_in in, axq_rows
 
 __global__ void __launch_bounds__(256) rows_layer_norm_kernel(axq_in in, const float *nw1, axq_rows_out out1, const float *nw2, axq_rows_out out2) {
     __shared__ float scratch[16];
-    const int t = blockIdx.x, k = in.k;
+    constexpr int NR = 4; // quads of a row that a thread keeps; wider rows are read again
+    const int t = blockIdx.x, k = in.k, tid = threadIdx.x, quads = out1.ldx >> 2;
     const float *x = in.x + (size_t)(in.rows ? in.rows[t] : t) * k;
+    f32x4 r[NR];
     float sum = 0.f, ss = 0.f;
-    for (int e = threadIdx.x; e < k; e += 256) sum += x[e];
+#pragma unroll
+    for (int i = 0; i < NR; i++) {
+        r[i] = tid + i * 256 < quads ? load_quad(x, (tid + i * 256) << 2, k) : f32x4{0.f, 0.f, 0.f, 0.f};
+        sum += (r[i][0] + r[i][1]) + (r[i][2] + r[i][3]);
+    }
+    for (int e = NR * 1024 + tid; e < k; e += 256) sum += x[e];
     const float mean = axq_block_sum(sum, scratch) / (float)k;
-    for (int e = threadIdx.x; e < k; e += 256) {
+#pragma unroll
+    for (int i = 0; i < NR; i++)
+#pragma unroll
+        for (int c = 0; c < 4; c++) {
+            const float d = ((tid + i * 256) << 2) + c < k ? r[i][c] - mean : 0.f;
+            ss = fmaf(d, d, ss);
+        }
+    for (int e = NR * 1024 + tid; e < k; e += 256) {
         const float d = x[e] - mean;
         ss = fmaf(d, d, ss);
     }
     const float inv = 1.0f / sqrtf(axq_block_sum(ss, scratch) / (float)k + in.eps);
-    for (int e = threadIdx.x; e < out1.ldx; e += 256) {
+#pragma unroll
+    for (int i = 0; i < NR; i++) {
+        const int q = tid + i * 256;
+        if (q >= quads) break;
+        const f32x4 n = (r[i] - mean) * inv; // past the end the weights are zeros
+        put_quad(out1, t, q << 2, n * load_quad(nw1, q << 2, k));
+        if (nw2) put_quad(out2, t, q << 2, n * load_quad(nw2, q << 2, k));
+    }
+    for (int e = NR * 1024 + tid; e < out1.ldx; e += 256) {
         const float n = e < k ? (x[e] - mean) * inv : 0.f;
         put(out1, t, e, e < k ? n * nw1[e] : 0.f);
         if (nw2) put(out2, t, e, e < k ? n * nw2[e] : 0.f);
@@ -731,6 +791,7 @@ int axq_rows_poly_norm(axq_ctx *ctx, const axq_in &in, int m, axq_rows_out out) 
 }
 
 int axq_rows_layer_norm(axq_ctx *ctx, const axq_in &in, int m, const float *nw1, axq_rows_out out1, const float *nw2, axq_rows_out out2) {
+    if (out1.ldx % 4) return axq_fail(ctx, AXQ_ERR_SHAPE_MISMATCH, "Shape mismatch: layer norms of rows %d apart", out1.ldx);
     if (nw2 && out2.ldx != out1.ldx) return axq_fail(ctx, AXQ_ERR_SHAPE_MISMATCH, "Shape mismatch: layer norms of rows %d and %d apart", out1.ldx, out2.ldx);
     rows_layer_norm_kernel<<<m, 256, 0, ctx->stream>>>(in, nw1, out1, nw2, out2);
     AXQ_LAUNCH_CHECK(ctx, "rows_layer_norm_kernel");

@@ -4,6 +4,8 @@
 
 namespace {
 
+typedef float f32x4 __attribute__((ext_vector_type(4)));
+
 // Best of the wave's candidates (value, index; index < 0: none), ties to the lower index.
 __device__ inline int wave_argmax(float v, int i) {
 #pragma unroll
@@ -15,7 +17,46 @@ __device__ inline int wave_argmax(float v, int i) {
     return __builtin_amdgcn_readfirstlane(i);
 }
 
-// One wave per row.
+__device__ inline float lane_of(float v, int lane) { return __builtin_bit_cast(float, __builtin_amdgcn_readlane(__builtin_bit_cast(int, v), lane)); }
+
+// Up to 64 experts: a wave per row, a lane per expert.  Places are counted: how many of the others come before this one.
+__global__ void __launch_bounds__(64) route_lanes_kernel(axq_moe_router r, const float *z, int ldz, int32_t *sel, float *wt) {
+    const int t = blockIdx.x, e = threadIdx.x, per = r.experts / r.groups, group = e / per;
+    float s = e < r.experts ? axq_sigmoid(z[(size_t)t * ldz + e]) : 0.f;
+    if (!(s == s)) s = 0.f; // with NaN among them places would not be distinct, and `sel` must hold experts whatever comes
+    bool usable = e < r.experts;
+    if (r.keep < r.groups) {
+        float a = 0.f, b = 0.f; // scores are positive; a group of one has no second
+        for (int j = 0; j < r.experts; j++) {
+            const float v = lane_of(s, j);
+            if (j / per == group) {
+                b = fmaxf(b, fminf(a, v));
+                a = fmaxf(a, v);
+            }
+        }
+        const float mine = a + b;
+        int before = 0;
+        for (int g = 0; g < r.groups; g++) {
+            const float v = lane_of(mine, g * per);
+            before += v > mine || (v == mine && g < group);
+        }
+        usable = usable && before < r.keep;
+    }
+    const uint64_t others = __builtin_amdgcn_ballot_w64(usable);
+    int before = 0;
+    for (int j = 0; j < r.experts; j++) {
+        const float v = lane_of(s, j);
+        before += ((others >> j) & 1) && (v > s || (v == s && j < e));
+    }
+    const bool chosen = usable && before < r.top;
+    const float inv = 1.0f / (axq_wave_sum(chosen ? s : 0.f) + 1e-20f);
+    if (chosen) {
+        sel[(size_t)t * r.top + before] = e;
+        wt[(size_t)t * r.top + before] = s * inv;
+    }
+}
+
+// Any number of experts: one wave per row.
 __global__ void __launch_bounds__(64) route_kernel(axq_moe_router r, const float *z, int ldz, int32_t *sel, float *wt) {
     __shared__ float score[AXQ_MOE_MAX_EXPERTS], group[AXQ_MOE_MAX_EXPERTS];
     __shared__ int chosen[AXQ_MOE_MAX_EXPERTS];
@@ -108,16 +149,21 @@ __global__ void __launch_bounds__(1024) sort_kernel(const int32_t *sel, int n, i
     }
 }
 
-__global__ void __launch_bounds__(256) combine_kernel(const float *ye, const int32_t *slot_of, const float *wt, int top, int width, float *y, axq_avg avg) {
-    const int t = blockIdx.x;
-    for (int e = blockIdx.y * 256 + threadIdx.x; e < width; e += 256 * gridDim.y) {
-        const size_t i = (size_t)t * width + e;
-        float s = 0.f;
-        for (int j = 0; j < top; j++) s = fmaf(wt[(size_t)t * top + j], ye[(size_t)slot_of[(size_t)t * top + j] * width + e], s);
-        const float v = y[i] + s;
-        y[i] = v;
-        if (avg.out) avg.out[i] = axq_average(avg, i, v);
-    }
+// V: f32x4 (widths that are multiples of 4) or float
+template <class V>
+__global__ void __launch_bounds__(256) combine_kernel(const V *ye, const int32_t *slot_of, const float *wt, int top, int width, V *y, axq_avg avg) {
+    const int t = blockIdx.x, e = blockIdx.y * 256 + threadIdx.x; // width, e: in units of V
+    if (e >= width) return;
+    const size_t i = (size_t)t * width + e;
+    V v = y[i];
+    for (int j = 0; j < top; j++) v += wt[(size_t)t * top + j] * ye[(size_t)slot_of[(size_t)t * top + j] * width + e];
+    y[i] = v;
+    if (!avg.out) return;
+    const V *past = reinterpret_cast<const V *>(avg.past);
+    const size_t stride = avg.stride / (sizeof(V) / 4);
+    V s = avg.w[avg.n] * v;
+    for (int j = 0; j < avg.n; j++) s += avg.w[j] * past[j * stride + i];
+    reinterpret_cast<V *>(avg.out)[i] = s;
 }
 
 } // namespace
@@ -126,7 +172,8 @@ int axq_moe_route(axq_ctx *ctx, const axq_moe_router &r, const float *z, int ldz
     if (r.experts < 1 || r.experts > AXQ_MOE_MAX_EXPERTS || r.groups < 1 || r.experts % r.groups || r.keep < 1 || r.keep > r.groups || r.top < 1 ||
         r.top > r.keep * (r.experts / r.groups) || m < 1)
         return axq_fail(ctx, AXQ_ERR_SHAPE_MISMATCH, "Shape mismatch: %d of %d experts, from %d of %d groups", r.top, r.experts, r.keep, r.groups);
-    route_kernel<<<m, 64, 0, ctx->stream>>>(r, z, ldz, sel, wt);
+    if (r.experts <= 64) route_lanes_kernel<<<m, 64, 0, ctx->stream>>>(r, z, ldz, sel, wt);
+    else route_kernel<<<m, 64, 0, ctx->stream>>>(r, z, ldz, sel, wt);
     AXQ_LAUNCH_CHECK(ctx, "route_kernel");
     return AXQ_OK;
 }
@@ -140,7 +187,10 @@ int axq_moe_sort(axq_ctx *ctx, const int32_t *sel, int n, int top, int experts, 
 }
 
 int axq_moe_combine(axq_ctx *ctx, const float *ye, const int32_t *slot_of, const float *wt, int top, int m, int width, float *y, const axq_avg &avg) {
-    combine_kernel<<<dim3(m, (width + 1023) / 1024), 256, 0, ctx->stream>>>(ye, slot_of, wt, top, width, y, avg);
+    if (width % 4 == 0) // (every row, and avg.stride = m rows, is then a whole number of them)
+        combine_kernel<f32x4><<<dim3(m, (width / 4 + 255) / 256), 256, 0, ctx->stream>>>(reinterpret_cast<const f32x4 *>(ye), slot_of, wt, top, width / 4,
+                                                                                         reinterpret_cast<f32x4 *>(y), avg);
+    else combine_kernel<float><<<dim3(m, (width + 255) / 256), 256, 0, ctx->stream>>>(ye, slot_of, wt, top, width, y, avg);
     AXQ_LAUNCH_CHECK(ctx, "combine_kernel");
     return AXQ_OK;
 }

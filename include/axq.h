@@ -289,10 +289,9 @@ typedef enum {
     AXQ_MIX_LIGHTNING = 1, /* linear attention: S <- decay S + k v^T, o = S^T q; SiLU on q, k, v; gated RMS norm over all heads */
     AXQ_MIX_WKV = 2,       /* time mixing: inputs leaning to the previous token's, a decay per token, head and key channel
                               (through decay_rank), a bonus for the current token, gated RMS norm per head */
-    AXQ_MIX_SOFTMAX = 3    /* causal softmax attention, score = q.k * scale, over the last `window` tokens and, with `pool` P, over
-                              one key and value per block of P tokens that lies wholly before the window, the means of its
-                              tokens'; rotary positions on the first rot_dims dimensions of q and k (neighbours paired);
-                              keys_as_values: values are the keys before rotation, there is no "mix.v"; head_gate: each
+    AXQ_MIX_SOFTMAX = 3    /* causal softmax attention, score = q.k * scale, over the last `window` tokens and, with `pool`, over the
+                              mean keys and values of the blocks of `pool` tokens that the window has left behind; rotary
+                              positions on the first rot_dims dimensions of q and k (neighbours paired); keys_as_values: values are the keys before rotation, there is no "mix.v"; head_gate: each
                               head's result times sigmoid of a product of its own, "mix.g" */
 } axq_mixer;
 /* Feed-forwards, of h = norm2(x) (ff > 0). */
@@ -338,8 +337,8 @@ typedef struct {
     int32_t norm;                           /* axq_norm_kind, of all norms of the residual stream */
     int32_t position_table;                 /* 1: "pos" is added to the embedding */
     int32_t parallel;                       /* 1: x + (mixer(norm1(x)) + ff(norm2(x))) instead of one after the other (layer norms only) */
-    int32_t depth_average;                  /* 1: after layer i, x <- sum over j <= i + 1 of "dwa"[j] X_j: X_0 the embedding, X_(j+1) layer
-                                               j's result before this (no loop) */
+    int32_t depth_average;                  /* 1: a layer hands on the sum of its own result, of all earlier layers' and of the embedding, weighted
+                                               by "dwa" (the embedding's weight first, its own last); not with a loop */
 } axq_stack_config;
 AXQ_API int axq_model_create_stack(axq_ctx *ctx, const axq_stack_config *cfg, axq_model **out);
 /* A tensor by name, from f32 values (host): layer -1 = "pos" [max_positions, width], "final.norm" [width] (tanh norm: and

@@ -56,8 +56,17 @@ def _gaps(s, router):
 
 
 def _router_classes(rng, router):
-    """Per expert and class: evenly spaced, in an order of its own for every class, without close calls."""
+    """Per expert and class: evenly spaced where they are few, in an order of its own for every class, without close calls."""
     n = router["experts"]
+    if n > 16:  # too many for even spacing: `top` of them high, in as many groups as are kept
+        groups = router.get("groups") or {"count": 1, "keep": 1}
+        out = []
+        for _ in range(CLASSES):
+            r, kept = rng.uniform(-0.45, -0.2, n), rng.permutation(groups["count"])[:groups["keep"]]
+            for i in range(router["top"]):
+                r[kept[i % len(kept)] * (n // groups["count"]) + 1 + 2 * (i // len(kept))] = rng.uniform(0.2, 0.45)
+            out.append(r)
+        return np.stack(out, axis=1)
     spaced, out = np.linspace(-0.45, 0.45, n) if n > 1 else np.zeros(1), []
     while len(out) < CLASSES:
         r = rng.permutation(spaced)

@@ -57,6 +57,9 @@ ONE_LAYER = {
     "mixture of one": one(mlp=gc.moe(groups=None, experts=1, top=1)),
     "one of many": one(mlp=gc.moe(groups=None, experts=7, top=1, shared=0)),
     "all of them": one(mlp=gc.moe(groups=None, experts=4, top=4)),
+    "mixture of 64": one(mlp=gc.moe(groups=(8, 2), experts=64, top=5, ff=9)),
+    "mixture of 96": one(mlp=gc.moe(groups=(8, 3), experts=96, top=6, ff=9)),
+    "mixture of 130 without groups": one(mlp=gc.moe(groups=None, experts=130, top=9, ff=5)),
     "mixture, wide experts": one(mlp=gc.moe(ff=130, shared=70), width=130),
     "mixture, narrow experts": one(mlp=gc.moe(ff=1, shared=1), width=40),
     "layers of different rotations, with and without feed-forward": gc.config([gc.attention(turn=gc.rot(20, 500.0, None)), gc.attention(mlp=gc.dense(24)),
