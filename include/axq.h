@@ -291,8 +291,8 @@ typedef enum {
                               (through decay_rank), a bonus for the current token, gated RMS norm per head */
     AXQ_MIX_SOFTMAX = 3    /* causal softmax attention, score = q.k * scale, over the last `window` tokens and, with `pool`, over the
                               mean keys and values of the blocks of `pool` tokens that the window has left behind; rotary
-                              positions on the first rot_dims dimensions of q and k (neighbours paired); keys_as_values: values are the keys before rotation, there is no "mix.v"; head_gate: each
-                              head's result times sigmoid of a product of its own, "mix.g" */
+                              positions on the first rot_dims dimensions of q and k (neighbours paired); keys_as_values: values are
+                              the keys before rotation, there is no "mix.v"; head_gate: each head's result times sigmoid of a product of its own, "mix.g" */
 } axq_mixer;
 /* Feed-forwards, of h = norm2(x) (ff > 0). */
 typedef enum {
